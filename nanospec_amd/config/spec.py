@@ -81,7 +81,8 @@ class AttentionSpec:
     sink: bool = False  # the soft-max's denominator holds one more term of score 0, which has no value
     own_kv: bool = True  # False: no key/value projections; the layer reads the cache of the run-order entry it names
     names: tuple[str, str, str, str] = ("q_proj.weight", "k_proj.weight", "v_proj.weight", "o_proj.weight")  # after the prefix
-    bias: bool = False  # the four projections have biases, named as their matrices plus ``bias_suffix``
+    bias: bool = False  # the four projections have biases, named as their matrices plus ``bias_suffix`` ...
+    out_bias: bool = True  # ... or, False, only those of q, k and v
     bias_suffix: str = ".b"
     # q (and k) pass an RMS norm over the WHOLE projection, all heads at once, with a weight per channel and this eps;
     # the weights are named as the q and k matrices plus ``whole_norm_suffix``
@@ -106,6 +107,7 @@ class AttentionSpec:
     # projection; W_g [heads * value size, hidden] is the tensor ``gate_name`` after the prefix and reads the mixer's input
     out_gate: bool = False
     gate_name: str = "g"
+    head_gate: bool = False  # the gate is one number per head instead: W_g [heads, hidden], head h's output times sigmoid(W_g h)_h
 
     @property
     def v_dim(self) -> int:
@@ -115,7 +117,7 @@ class AttentionSpec:
     def general(self) -> bool:
         return bool(self.value_dim not in (0, self.head_dim) or self.qk_norm_eps is not None or self.score_cap or self.chunk or self.sink
                     or not self.own_kv or self.bias or self.whole_norm_eps is not None or self.slope_exp or self.value_mix
-                    or self.head_norm_eps is not None or self.value_is_key or self.sink_name or self.out_gate)
+                    or self.head_norm_eps is not None or self.value_is_key or self.sink_name or self.out_gate or self.head_gate)
 
 
 @dataclass(frozen=True)
@@ -219,9 +221,77 @@ class RetentionSpec:
 
 
 @dataclass(frozen=True)
+class GatedLinearSpec:
+    """Gated linear attention: linear attention whose decay, one per token, head and key channel, the input chooses.  With h the
+    input, per head: q = W_q h * query_scale, k = W_k h [key_dim], v = W_v h [value_dim], alpha = sigmoid(W_a2 (W_a1 h) + b)^(1/tau)
+    [key_dim];  S [key_dim, value_dim] starts at zero:
+        S_t = diag(alpha_t) S_(t-1) + k_t v_t^T;   o_t = S_t^T q_t
+    then o / rms(o) per head (``norm_eps``) times a weight [value_dim] that all heads share, times silu(W_g h), through W_o.
+    Decays, state and read-out are 32-bit.  ``decay_rank``: inner size of the decay's two matrices, read from the checkpoint when
+    None (random weights need it given).  ``names``: q, k, v, the gate, o, the norm's weight, a1, a2 after the prefix; the bias is
+    a2's name plus ``bias_suffix``."""
+
+    kind: ClassVar[str] = "gated_linear"
+    hidden: int
+    heads: int
+    key_dim: int
+    value_dim: int
+    tau: float
+    query_scale: float
+    norm_eps: float
+    decay_rank: int | None = None
+    names: tuple = ("q", "k", "v", "g", "o", "norm", "a1", "a2")
+    bias_suffix: str = ".b"
+
+
+@dataclass(frozen=True)
+class SelectiveScanSpec:
+    """The selective scan of Mamba.  With h the input: [x | z] = W_in h (``inner`` each); x passes a causal convolution of ``conv``
+    taps per channel with a bias, and a SiLU; [r | B | C] = W_x x (``dt_rank``, ``state``, ``state``); dt = softplus(W_dt r + b_dt)
+    [inner]; A = -exp(A_log) [inner, state].  Per channel c and state n, S from zero:
+        S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;   y_c = sum_n S[c, n] C_n + D_c x_c
+    then y * silu(z) through W_o.  Step sizes, decays, state and read-out are 32-bit.  ``names``: in, conv, x, dt, A_log, D, o after
+    the prefix; the two biases are the convolution's and dt's names plus ``bias_suffix``."""
+
+    kind: ClassVar[str] = "selective_scan"
+    hidden: int
+    inner: int
+    state: int
+    dt_rank: int
+    conv: int
+    names: tuple = ("in", "conv", "x", "dt", "A_log", "D", "o")
+    bias_suffix: str = ".b"
+
+
+@dataclass(frozen=True)
+class StateSpaceSpec:
+    """The state-space recurrence of Mamba-2, one decay per token and head.  With h the input and inner = heads * value_dim:
+    [z: inner | x: inner | B: groups * state | C: groups * state | dt: heads] = W_in h; x, B and C together pass a causal convolution of
+    ``conv`` taps per channel with a bias, and a SiLU; dt = softplus(dt + dt_bias).  Per head (B and C of group h // (heads /
+    groups)), S [state, value_dim] from zero:
+        S_t = exp(-exp(A_log_h) dt) S_(t-1) + dt B_t x_t^T;   y_t = S_t^T C_t + D_h x_t
+    then y * silu(z), an RMS norm in ``norm_groups`` equal parts (``norm_eps``) times a weight [inner], through W_o.  Step sizes,
+    decays, state and read-out are 32-bit.  ``names``: in, conv, dt_bias, A_log, D, norm, o after the prefix; the convolution's
+    bias is its name plus ``bias_suffix``."""
+
+    kind: ClassVar[str] = "state_space"
+    hidden: int
+    heads: int
+    value_dim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int
+    norm_eps: float
+    names: tuple = ("in", "conv", "dt_bias", "A_log", "D", "norm", "o")
+    bias_suffix: str = ".b"
+
+
+@dataclass(frozen=True)
 class ParallelMixerSpec:
     """Two mixers side by side that read the same input: left_scale * left(h) + right_scale * right(h).  Each keeps what it
-    keeps (pages, state); their tensors lie under the two prefixes."""
+    keeps (pages, state); their tensors lie under the two prefixes.  ``out_norm_eps``: each output first passes an RMS norm over
+    the width with this eps and the weight ``out_norm_names`` (left, right, after the mixer's prefix)."""
 
     kind: ClassVar[str] = "parallel"
     left: object
@@ -229,6 +299,8 @@ class ParallelMixerSpec:
     left_scale: float = 1.0
     right_scale: float = 1.0
     prefixes: tuple[str, str] = ("left.", "right.")
+    out_norm_eps: float | None = None
+    out_norm_names: tuple[str, str] = ("left.out", "right.out")
 
 
 @dataclass(frozen=True)
@@ -273,7 +345,11 @@ class MoESpec:
     experts of the ``keep_groups`` best groups can be chosen.  ``shared_gate_name``: the shared expert's output is multiplied by
     sigmoid(w h), one number per token, w [1, hidden] this tensor after the shared prefix ("" for none).  The soft-max over the
     chosen logits is the soft-max over all logits divided by the chosen ones' sum.  Experts of the form ``PlainFFSpec`` have no gate
-    matrix."""
+    matrix.
+    ``score`` = "softmax_all": the scores are s = soft-max over all logits; the choice goes by s + correction and the weights are
+    the chosen experts' s divided by their sum (+ 1e-20).  ``group_best`` = 1: a group's score is its largest choice score alone.
+    ``weight_scale`` multiplies the weights, whatever the scores.  ``identity``: so many more outputs of the router, behind the
+    experts' (and in the groups and the soft-max with them), are experts without tensors whose output is the input itself."""
 
     kind: ClassVar[str] = "moe"
     hidden: int
@@ -291,6 +367,9 @@ class MoESpec:
     groups: int = 1
     keep_groups: int = 1
     shared_gate_name: str = ""
+    group_best: int = 2
+    weight_scale: float = 1.0
+    identity: int = 0
 
 
 @dataclass(frozen=True)

@@ -30,6 +30,8 @@ __device__ __forceinline__ float activation_of(float z, int act) {
   return r * r;
 }
 
+__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = NS_WAVE / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, NS_WAVE);

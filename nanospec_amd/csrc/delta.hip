@@ -15,32 +15,35 @@
 #define ND_ROWS 16  // key channels of a column that one thread owns
 
 // ------------------------------------------------------------------------------------------------
-// y[r][c] = silu(sum_j taps[c][j] * in(i - (K-1) + j)),  i the token's index among its request's tokens of this step;
-// in(t) is this step's input for t >= 0 and the carried input K-1+t for t < 0.
+// y[r][c] = silu(bias[c] + sum_j taps[c][j] * in(i - (K-1) + j)),  i the token's index among its request's tokens of this step;
+// in(t) is this step's input for t >= 0 and the carried input K-1+t for t < 0.  ``bias`` may be null.  ``copy`` (or null)
+// receives y in the type of the input as well, for a product that reads it.
 // ------------------------------------------------------------------------------------------------
 template <typename T>
-__global__ void conv_silu_kernel(float* __restrict__ out, const T* __restrict__ x, int x_stride, const float* __restrict__ taps,
-                                 const float* __restrict__ state, size_t slot_stride, size_t conv_off, const int* __restrict__ token_req,
+__global__ void conv_silu_kernel(float* __restrict__ out, T* __restrict__ copy, const T* __restrict__ x, int x_stride,
+                                 const float* __restrict__ taps, const float* __restrict__ bias, const float* __restrict__ state, size_t slot_stride, size_t conv_off, const int* __restrict__ token_req,
                                  const int* __restrict__ qo_indptr, const int* __restrict__ state_slots, int C, int K) {
   const int r = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int b = token_req[r];
   const int i = r - qo_indptr[b];
   const float* carried = state + (size_t)state_slots[b] * slot_stride + conv_off;
-  float y = 0.f;
+  float y = bias ? bias[c] : 0.f;
   for (int j = 0; j < K; ++j) {
     const int t = i - (K - 1) + j;
     const float v = t >= 0 ? to_f(x[(size_t)(r - (K - 1) + j) * x_stride + c]) : carried[(size_t)(K - 1 + t) * C + c];
     y = fmaf(taps[(size_t)c * K + j], v, y);
   }
-  out[(size_t)r * C + c] = y / (1.f + expf(-y));
+  y = y / (1.f + expf(-y));
+  out[(size_t)r * C + c] = y;
+  if (copy) copy[(size_t)r * C + c] = from_f<T>(y);
 }
 
 // The same for four neighbouring channels a thread, with 16-byte accesses to taps, carried inputs and results, for the
 // usual numbers of taps (so that the taps are registers) and channels that are a multiple of four.
 template <typename T, int K>
-__global__ void conv_silu_vec_kernel(float* __restrict__ out, const T* __restrict__ x, int x_stride, const float* __restrict__ taps,
-                                     const float* __restrict__ state, size_t slot_stride, size_t conv_off, const int* __restrict__ token_req,
+__global__ void conv_silu_vec_kernel(float* __restrict__ out, T* __restrict__ copy, const T* __restrict__ x, int x_stride,
+                                     const float* __restrict__ taps, const float* __restrict__ bias, const float* __restrict__ state, size_t slot_stride, size_t conv_off, const int* __restrict__ token_req,
                                      const int* __restrict__ qo_indptr, const int* __restrict__ state_slots, int C) {
   typedef T vec_t __attribute__((ext_vector_type(4)));
   const int r = blockIdx.x, c = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
@@ -55,6 +58,10 @@ __global__ void conv_silu_vec_kernel(float* __restrict__ out, const T* __restric
     tp[4 * e] = t.x, tp[4 * e + 1] = t.y, tp[4 * e + 2] = t.z, tp[4 * e + 3] = t.w;
   }
   float y[4] = {0.f, 0.f, 0.f, 0.f};
+  if (bias) {
+    const float4 bv = *reinterpret_cast<const float4*>(bias + c);
+    y[0] = bv.x, y[1] = bv.y, y[2] = bv.z, y[3] = bv.w;
+  }
 #pragma unroll
   for (int j = 0; j < K; ++j) {
     const int t = i - (K - 1) + j;
@@ -74,6 +81,10 @@ __global__ void conv_silu_vec_kernel(float* __restrict__ out, const T* __restric
   res.x = y[0] / (1.f + expf(-y[0])), res.y = y[1] / (1.f + expf(-y[1]));
   res.z = y[2] / (1.f + expf(-y[2])), res.w = y[3] / (1.f + expf(-y[3]));
   *reinterpret_cast<float4*>(out + (size_t)r * C + c) = res;
+  if (copy) {
+    const vec_t cv = {from_f<T>(res.x), from_f<T>(res.y), from_f<T>(res.z), from_f<T>(res.w)};
+    *reinterpret_cast<vec_t*>(copy + (size_t)r * C + c) = cv;
+  }
 }
 
 // After the convolution has read them: the carried inputs become the last K-1 inputs including this step's.
@@ -93,7 +104,7 @@ __global__ void conv_carry_kernel(const T* __restrict__ x, int x_stride, float* 
   }
 }
 
-extern "C" int ns_conv_silu_carry(float* out, const void* x, int x_stride, const float* taps, float* state, size_t slot_stride,
+extern "C" int ns_conv_silu_carry(float* out, void* copy, const void* x, int x_stride, const float* taps, const float* bias, float* state, size_t slot_stride,
                                   size_t conv_off, const int* token_req, const int* qo_indptr, const int* state_slots, int n_tokens,
                                   int n_reqs, int C, int K, int dtype, hipStream_t stream) {
   if (n_tokens <= 0 || n_reqs <= 0 || n_reqs > 65535 || C <= 0 || K < 1 || K > ND_MAX_TAPS) return NS_ERR_BAD_ARG;
@@ -102,16 +113,17 @@ extern "C" int ns_conv_silu_carry(float* out, const void* x, int x_stride, const
   if (bx > 65535) return NS_ERR_BAD_ARG;
   const size_t esize = dtype == NS_DTYPE_F32 ? 4 : 2;
   const bool vec = C % 4 == 0 && x_stride % 4 == 0 && ((uintptr_t)x % (4 * esize)) == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)taps % 16) == 0 &&
+                   ((uintptr_t)bias % 16) == 0 && ((uintptr_t)copy % (4 * esize)) == 0 &&
                    ((uintptr_t)state % 16) == 0 && slot_stride % 4 == 0 && conv_off % 4 == 0 && K >= 2 && K <= 4;
   if (vec) {
     dim3 grid(n_tokens, (C / 4 + 255) / 256);
 #define ND_CONV(KK)                                                                                                                         \
   case KK:                                                                                                                                  \
     if (dtype == NS_DTYPE_F32)                                                                                                              \
-      conv_silu_vec_kernel<float, KK><<<grid, 256, 0, stream>>>(out, (const float*)x, x_stride, taps, state, slot_stride, conv_off, token_req, \
+      conv_silu_vec_kernel<float, KK><<<grid, 256, 0, stream>>>(out, (float*)copy, (const float*)x, x_stride, taps, bias, state, slot_stride, conv_off, token_req, \
                                                                 qo_indptr, state_slots, C);                                                \
     else                                                                                                                                    \
-      conv_silu_vec_kernel<bf16_t, KK><<<grid, 256, 0, stream>>>(out, (const bf16_t*)x, x_stride, taps, state, slot_stride, conv_off, token_req, \
+      conv_silu_vec_kernel<bf16_t, KK><<<grid, 256, 0, stream>>>(out, (bf16_t*)copy, (const bf16_t*)x, x_stride, taps, bias, state, slot_stride, conv_off, token_req, \
                                                                  qo_indptr, state_slots, C);                                               \
     break
     switch (K) {
@@ -123,10 +135,10 @@ extern "C" int ns_conv_silu_carry(float* out, const void* x, int x_stride, const
   } else {
     dim3 grid(n_tokens, bx);
     if (dtype == NS_DTYPE_F32)
-      conv_silu_kernel<float><<<grid, 256, 0, stream>>>(out, (const float*)x, x_stride, taps, state, slot_stride, conv_off, token_req,
+      conv_silu_kernel<float><<<grid, 256, 0, stream>>>(out, (float*)copy, (const float*)x, x_stride, taps, bias, state, slot_stride, conv_off, token_req,
                                                          qo_indptr, state_slots, C, K);
     else
-      conv_silu_kernel<bf16_t><<<grid, 256, 0, stream>>>(out, (const bf16_t*)x, x_stride, taps, state, slot_stride, conv_off, token_req,
+      conv_silu_kernel<bf16_t><<<grid, 256, 0, stream>>>(out, (bf16_t*)copy, (const bf16_t*)x, x_stride, taps, bias, state, slot_stride, conv_off, token_req,
                                                           qo_indptr, state_slots, C, K);
   }
   if (K > 1) {
@@ -143,8 +155,6 @@ extern "C" int ns_conv_silu_carry(float* out, const void* x, int x_stride, const
 // Per token: q and k of every key/value head become unit vectors, x / sqrt(sum(x^2) + 1e-6), q times D^(-1/2), in
 // place in qkv [n][2 G D + H E]; g = exp(-exp(A_log[h]) softplus(a + dt_bias)) [n][H D]; beta = sigmoid(b) [n][H].
 // ------------------------------------------------------------------------------------------------
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-
 // grid (tokens, Y): the first ceil(2 G / 4) blocks of a token take one vector a wave; the others 1,024 decays each (and
 // the first of them the write strengths), so that no wave walks through a chain of dependent loads.
 template <typename T>
@@ -426,38 +436,42 @@ extern "C" int ns_delta_scan(float* o, const float* qkv, int C, const float* g, 
 
 // ------------------------------------------------------------------------------------------------
 // out[r][h][:] = o / sqrt(mean(o^2) + eps) * w[:] * sigmoid(gate[r][h][:]),  o float, gate and out in the model's type.
+// ``gate_first``: the gate stands in front of the norm, x = o * gate, out = x / sqrt(mean(x^2) + eps) * w[:].
 // ------------------------------------------------------------------------------------------------
 template <typename T>
 __global__ void gated_rms_kernel(T* __restrict__ out, const float* __restrict__ o, const T* __restrict__ gate, int gate_stride,
-                                 const float* __restrict__ w, int w_stride, const float* __restrict__ den, int H, int E, float eps, int silu) {
+                                 const float* __restrict__ w, int w_stride, const float* __restrict__ den, int H, int E, float eps, int silu,
+                                 int gate_first) {
   __shared__ float scratch[16];
   const int r = blockIdx.x, h = blockIdx.y;
   if (w) w += (size_t)h * w_stride;  // 0: all heads share one weight; no weight at all: the factor is 1
   const float* p = o + ((size_t)r * H + h) * E;
   const float dinv = den ? 1.f / den[(size_t)r * H + h] : 1.f;  // a head's read-out that comes undivided
+  // the gate: sigmoid(z), or with ``silu`` z sigmoid(z)
+  auto gate_of = [&](int e) {
+    const float z = to_f(gate[(size_t)r * gate_stride + (size_t)h * E + e]);
+    return (silu ? z : 1.f) / (1.f + expf(-z));
+  };
   float ss = 0.f;
   for (int e = threadIdx.x; e < E; e += blockDim.x) {
-    const float v = p[e] * dinv;
+    const float v = p[e] * dinv * (gate_first ? gate_of(e) : 1.f);
     ss = fmaf(v, v, ss);
   }
   ss = blockDim.x > NS_WAVE ? block_sum(ss, scratch) : wave_sum(ss);
   const float rinv = 1.f / sqrtf(ss / (float)E + eps);
-  for (int e = threadIdx.x; e < E; e += blockDim.x) {
-    const float z = to_f(gate[(size_t)r * gate_stride + (size_t)h * E + e]);
-    // the gate: sigmoid(z), or with ``silu`` z sigmoid(z)
-    out[((size_t)r * H + h) * E + e] = from_f<T>(p[e] * dinv * rinv * (w ? w[e] : 1.f) * (silu ? z : 1.f) / (1.f + expf(-z)));
-  }
+  for (int e = threadIdx.x; e < E; e += blockDim.x)
+    out[((size_t)r * H + h) * E + e] = from_f<T>(p[e] * dinv * rinv * (w ? w[e] : 1.f) * gate_of(e));
 }
 
 extern "C" int ns_gated_rms(void* out, const float* o, const void* gate, int gate_stride, const float* w, int w_stride, const float* den,
-                            int n_tokens, int H, int E, float eps, int silu, int dtype, hipStream_t stream) {
+                            int n_tokens, int H, int E, float eps, int silu, int gate_first, int dtype, hipStream_t stream) {
   if (n_tokens <= 0 || H <= 0 || H > 65535 || E <= 0) return NS_ERR_BAD_ARG;
   dim3 grid(n_tokens, H);
   const int threads = E > 512 ? 256 : NS_WAVE;  // a wave a head, four for wide heads (all heads normed as one)
   if (dtype == NS_DTYPE_F32)
-    gated_rms_kernel<float><<<grid, threads, 0, stream>>>((float*)out, o, (const float*)gate, gate_stride, w, w_stride, den, H, E, eps, silu);
+    gated_rms_kernel<float><<<grid, threads, 0, stream>>>((float*)out, o, (const float*)gate, gate_stride, w, w_stride, den, H, E, eps, silu, gate_first);
   else if (dtype == NS_DTYPE_BF16)
-    gated_rms_kernel<bf16_t><<<grid, threads, 0, stream>>>((bf16_t*)out, o, (const bf16_t*)gate, gate_stride, w, w_stride, den, H, E, eps, silu);
+    gated_rms_kernel<bf16_t><<<grid, threads, 0, stream>>>((bf16_t*)out, o, (const bf16_t*)gate, gate_stride, w, w_stride, den, H, E, eps, silu, gate_first);
   else
     return NS_ERR_UNSUPPORTED;
   return ns_launch_status();

@@ -9,6 +9,8 @@
 // The experts' matrices are stacked: gate and up [experts][ff][W], down [experts][W][ff].
 // More rows may stand below the experts' in the router's matrix (a shared expert's gate): their logits are formed and kept
 // beside the experts' and have no part in the choice.
+// The last outputs of a router may be identity experts, which have no matrices: what such a pair adds is its weight times the
+// input row, formed where the pairs are added up (``moe_combine``); the experts' kernels leave these pairs out.
 #include "common.h"
 
 #define MOE_MAX_EXPERTS 1024
@@ -101,11 +103,17 @@ __global__ __launch_bounds__(256) void moe_logits_few_kernel(const T* __restrict
 // A wave a token: the choice scores in LDS, every lane looks through its share for the largest one not yet taken, the lanes'
 // candidates meet by lane exchange (the larger value wins, the lower index among equals; what is no number counts as
 // minus infinity, so a row of anything still chooses ``top`` different experts).
-// ``sigmoid`` = 0: the choice goes by the logits and the weights are the soft-max over the chosen logits.
-// ``sigmoid`` = 1: scores s = sigmoid(z); the choice goes by s + correction[e] (``correction`` may be null) and the weights are
-// the chosen experts' s, not renormalized.  ``groups`` > 1: the experts form that many equal groups of neighbours; a group's
-// score is the sum of its two largest choice scores (of its one, if it has one), and only the ``keep`` best groups' experts
-// can be chosen: the others never enter the comparison, whatever their scores' sign.
+// ``score`` = MOE_CHOSEN_SOFTMAX: the choice goes by the logits and the weights are the soft-max over the chosen logits.
+// ``score`` = MOE_SIGMOID: scores s = sigmoid(z); the choice goes by s + correction[e] (``correction`` may be null) and the
+// weights are the chosen experts' s, not renormalized.
+// ``score`` = MOE_SOFTMAX: scores s = soft-max over all logits; the choice goes by s + correction[e], the weights are the chosen
+// experts' s divided by their sum (+ 1e-20).
+// All weights are then multiplied by ``scale``.  ``groups`` > 1: the experts form that many equal groups of neighbours; a
+// group's score is the sum of its ``group_best`` (1 or 2) largest choice scores (of its one, if it has one), and only the
+// ``keep`` best groups' experts can be chosen: the others never enter the comparison, whatever their scores' sign.
+#define MOE_CHOSEN_SOFTMAX 0
+#define MOE_SIGMOID 1
+#define MOE_SOFTMAX 2
 __device__ __forceinline__ void wave_best(float& bv, int& best) {
 #pragma unroll
   for (int o = NS_WAVE / 2; o > 0; o >>= 1) {
@@ -116,23 +124,27 @@ __device__ __forceinline__ void wave_best(float& bv, int& best) {
 }
 
 __global__ __launch_bounds__(64) void moe_choose_kernel(const float* __restrict__ z, int z_stride, int* __restrict__ sel, float* __restrict__ wt,
-                                                        int n, int experts, int top, int sigmoid, const float* __restrict__ correction, int groups,
-                                                        int keep) {
+                                                        int n, int experts, int top, int score, const float* __restrict__ correction, int groups,
+                                                        int keep, int group_best, float scale) {
   __shared__ float zs[MOE_MAX_EXPERTS];   // choice scores
   __shared__ float ws[MOE_MAX_EXPERTS];   // what the weights are made from: the logits, or the sigmoid scores
   __shared__ float gs[MOE_MAX_EXPERTS];   // group scores
   __shared__ unsigned char taken[MOE_MAX_EXPERTS];
   __shared__ unsigned char gkept[MOE_MAX_EXPERTS];
   const int t = blockIdx.x, lane = threadIdx.x;
+  float zmax = -INFINITY, zsum = 0.f;  // of the soft-max over all logits
+  if (score == MOE_SOFTMAX) {
+    for (int e = lane; e < experts; e += NS_WAVE) zmax = fmaxf(zmax, z[(size_t)t * z_stride + e]);
+    zmax = wave_max(zmax);
+    for (int e = lane; e < experts; e += NS_WAVE) zsum += expf(z[(size_t)t * z_stride + e] - zmax);
+    zsum = wave_sum(zsum);
+  }
   for (int e = lane; e < experts; e += NS_WAVE) {
     float v = z[(size_t)t * z_stride + e];
-    if (sigmoid) {
-      v = 1.f / (1.f + expf(-v));
-      ws[e] = v;
-      if (correction) v += correction[e];
-    } else {
-      ws[e] = v;
-    }
+    if (score == MOE_SIGMOID) v = 1.f / (1.f + expf(-v));
+    else if (score == MOE_SOFTMAX) v = expf(v - zmax) / zsum;
+    ws[e] = v;
+    if (correction) v += correction[e];
     zs[e] = v == v ? v : -INFINITY;
     taken[e] = 0;
   }
@@ -146,7 +158,7 @@ __global__ __launch_bounds__(64) void moe_choose_kernel(const float* __restrict_
         if (v > a) b = a, a = v;
         else if (v > b) b = v;
       }
-      gs[g] = per > 1 ? a + b : a;
+      gs[g] = per > 1 && group_best > 1 ? a + b : a;
       gkept[g] = 0;
     }
     __syncthreads();
@@ -173,7 +185,7 @@ __global__ __launch_bounds__(64) void moe_choose_kernel(const float* __restrict_
     wave_best(bv, best);
     if (lane == 0) taken[best] = 1;
     float w;
-    if (sigmoid) {
+    if (score != MOE_CHOSEN_SOFTMAX) {
       w = ws[best];
     } else {
       if (k == 0) largest = bv;
@@ -185,15 +197,17 @@ __global__ __launch_bounds__(64) void moe_choose_kernel(const float* __restrict_
   }
   if (lane < top) {
     sel[(size_t)t * top + lane] = mine_idx;
-    wt[(size_t)t * top + lane] = sigmoid ? mine : mine / sum;
+    wt[(size_t)t * top + lane] = (score == MOE_SIGMOID ? mine : mine / (score == MOE_SOFTMAX ? sum + 1e-20f : sum)) * scale;
   }
 }
 
 // ``z``: float32 [n][experts + extra]; ``extra``: rows of ``wr`` (and ``br``) below the experts'
 extern "C" int ns_moe_route(const void* h, int h_stride, const float* wr, const float* br, float* z, int* sel, float* wt, int n, int W, int experts,
-                            int extra, int top, int sigmoid, const float* correction, int groups, int keep, int dtype, hipStream_t stream) {
+                            int extra, int top, int score, const float* correction, int groups, int keep, int group_best, float scale, int dtype,
+                            hipStream_t stream) {
   if (n <= 0 || W <= 0 || experts <= 0 || experts > MOE_MAX_EXPERTS || top <= 0 || top > MOE_MAX_TOP || top > experts) return NS_ERR_BAD_ARG;
-  if (extra < 0) return NS_ERR_BAD_ARG;
+  if (extra < 0 || score < MOE_CHOSEN_SOFTMAX || score > MOE_SOFTMAX || (correction && score == MOE_CHOSEN_SOFTMAX) || group_best < 1 || group_best > 2)
+    return NS_ERR_BAD_ARG;
   const int rows = experts + extra;
   if (groups < 1 || experts % groups || keep < 1 || keep > groups || top > keep * (experts / groups)) return NS_ERR_BAD_ARG;
   dim3 grid((n + ROUTE_TOK - 1) / ROUTE_TOK, (rows + 3) / 4);
@@ -210,7 +224,7 @@ extern "C" int ns_moe_route(const void* h, int h_stride, const float* wr, const 
     moe_logits_kernel<float><<<grid, 256, 0, stream>>>((const float*)h, h_stride, wr, br, z, n, W, rows, vec);
   else
     moe_logits_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)h, h_stride, wr, br, z, n, W, rows, vec);
-  moe_choose_kernel<<<n, 64, 0, stream>>>(z, rows, sel, wt, n, experts, top, sigmoid, correction, groups, keep);
+  moe_choose_kernel<<<n, 64, 0, stream>>>(z, rows, sel, wt, n, experts, top, score, correction, groups, keep, group_best, scale);
   return ns_launch_status();
 }
 
@@ -264,11 +278,12 @@ __device__ __forceinline__ float row_dot(const T* __restrict__ w, const float* _
 
 template <typename T>
 __global__ __launch_bounds__(256) void moe_rows_up_kernel(const T* __restrict__ h, int h_stride, const T* __restrict__ wg, const T* __restrict__ wu,
-                                                          const int* __restrict__ sel, float* __restrict__ act, int W, int ff, int top, int per,
+                                                          const int* __restrict__ sel, float* __restrict__ act, int W, int ff, int experts, int top, int per,
                                                           float limit, float alpha, float shift, int act_kind, int vec) {
   extern __shared__ __attribute__((aligned(16))) float moe_lds[];  // [W]
   const int t = blockIdx.z, k = blockIdx.y, lane = threadIdx.x % NS_WAVE, wave = threadIdx.x / NS_WAVE, waves = blockDim.x / NS_WAVE;
   const int e = sel[(size_t)t * top + k];
+  if (e >= experts) return;  // an identity expert
   for (int c = threadIdx.x; c < W; c += blockDim.x) moe_lds[c] = to_f(h[(size_t)t * h_stride + c]);
   __syncthreads();
   const int f0 = blockIdx.x * per, f1 = min(ff, f0 + per);
@@ -283,11 +298,12 @@ __global__ __launch_bounds__(256) void moe_rows_up_kernel(const T* __restrict__ 
 
 template <typename T>
 __global__ __launch_bounds__(256) void moe_rows_down_kernel(const float* __restrict__ act, const T* __restrict__ wd, const int* __restrict__ sel,
-                                                            const float* __restrict__ wt, float* __restrict__ out, int W, int ff, int top, int per,
-                                                            int vec) {
+                                                            const float* __restrict__ wt, float* __restrict__ out, int W, int ff, int experts, int top,
+                                                            int per, int vec) {
   extern __shared__ __attribute__((aligned(16))) float moe_lds[];  // [ff]
   const int t = blockIdx.z, k = blockIdx.y, lane = threadIdx.x % NS_WAVE, wave = threadIdx.x / NS_WAVE, waves = blockDim.x / NS_WAVE;
   const int e = sel[(size_t)t * top + k];
+  if (e >= experts) return;
   const float share = wt[(size_t)t * top + k];
   for (int f = threadIdx.x; f < ff; f += blockDim.x) moe_lds[f] = act[((size_t)t * top + k) * ff + f];
   __syncthreads();
@@ -306,10 +322,10 @@ static int moe_slice(int channels, int rows) {
 }
 
 extern "C" int ns_moe_expert_rows(const void* h, int h_stride, const void* wg, const void* wu, const void* wd, const int* sel, const float* wt,
-                                  float* act, float* out, int n, int W, int ff, int top, float limit, float alpha, float shift, int act_kind,
-                                  int dtype, hipStream_t stream) {
+                                  float* act, float* out, int n, int W, int ff, int top, int experts, float limit, float alpha, float shift,
+                                  int act_kind, int dtype, hipStream_t stream) {
   if (!wg && (act_kind < 0 || act_kind >= NS_ACTIVATIONS)) return NS_ERR_BAD_ARG;
-  if (n <= 0 || n > 65535 || W <= 0 || ff <= 0 || top <= 0 || top > 65535) return NS_ERR_BAD_ARG;
+  if (n <= 0 || n > 65535 || W <= 0 || ff <= 0 || top <= 0 || top > 65535 || experts <= 0) return NS_ERR_BAD_ARG;
   if ((size_t)W * sizeof(float) > 64 * 1024 || (size_t)ff * sizeof(float) > 64 * 1024) return NS_ERR_UNSUPPORTED;
   const size_t elem = dtype == NS_DTYPE_F32 ? 4 : 2;
   const int vec_up = W % 8 == 0 && (uintptr_t)wg % (8 * elem) == 0 && (uintptr_t)wu % (8 * elem) == 0;
@@ -318,12 +334,12 @@ extern "C" int ns_moe_expert_rows(const void* h, int h_stride, const void* wg, c
   dim3 g1((ff + per_f - 1) / per_f, top, n), g2((W + per_c - 1) / per_c, top, n);
   if (dtype == NS_DTYPE_F32) {
     moe_rows_up_kernel<float><<<g1, 256, W * sizeof(float), stream>>>((const float*)h, h_stride, (const float*)wg, (const float*)wu, sel, act, W, ff,
-                                                                       top, per_f, limit, alpha, shift, act_kind, vec_up);
-    moe_rows_down_kernel<float><<<g2, 256, ff * sizeof(float), stream>>>(act, (const float*)wd, sel, wt, out, W, ff, top, per_c, vec_down);
+                                                                       experts, top, per_f, limit, alpha, shift, act_kind, vec_up);
+    moe_rows_down_kernel<float><<<g2, 256, ff * sizeof(float), stream>>>(act, (const float*)wd, sel, wt, out, W, ff, experts, top, per_c, vec_down);
   } else if (dtype == NS_DTYPE_BF16) {
     moe_rows_up_kernel<bf16_t><<<g1, 256, W * sizeof(float), stream>>>((const bf16_t*)h, h_stride, (const bf16_t*)wg, (const bf16_t*)wu, sel, act, W,
-                                                                        ff, top, per_f, limit, alpha, shift, act_kind, vec_up);
-    moe_rows_down_kernel<bf16_t><<<g2, 256, ff * sizeof(float), stream>>>(act, (const bf16_t*)wd, sel, wt, out, W, ff, top, per_c, vec_down);
+                                                                        ff, experts, top, per_f, limit, alpha, shift, act_kind, vec_up);
+    moe_rows_down_kernel<bf16_t><<<g2, 256, ff * sizeof(float), stream>>>(act, (const bf16_t*)wd, sel, wt, out, W, ff, experts, top, per_c, vec_down);
   } else {
     return NS_ERR_UNSUPPORTED;
   }
@@ -357,7 +373,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
   __shared__ int cnt[MOE_MAX_EXPERTS], off[MOE_MAX_EXPERTS], cur[MOE_MAX_EXPERTS];
   for (int e = threadIdx.x; e < experts; e += blockDim.x) cnt[e] = 0, cur[e] = 0;
   __syncthreads();
-  for (int p = threadIdx.x; p < pairs; p += blockDim.x) atomicAdd(&cnt[sel[p]], 1);
+  for (int p = threadIdx.x; p < pairs; p += blockDim.x)
+    if (sel[p] < experts) atomicAdd(&cnt[sel[p]], 1);  // (pairs of identity experts have no place)
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0, tiles = 0;
@@ -373,7 +390,7 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
   // (which pair of an expert gets which of its places depends on timing; a pair's result does not depend on its place)
   for (int p = threadIdx.x; p < pairs; p += blockDim.x) {
     const int e = sel[p];
-    perm[off[e] + atomicAdd(&cur[e], 1)] = p;
+    if (e < experts) perm[off[e] + atomicAdd(&cur[e], 1)] = p;
   }
 }
 
@@ -546,29 +563,44 @@ extern "C" int ns_clipped_glu(void* out, const void* gu, int gu_stride, int n, i
   return ns_launch_status();
 }
 
+// What the outputs of a router beyond the experts do: a pair (t, k) with sel[t][k] >= experts adds its weight times the input row.
+struct MoeIdentity {
+  const int* sel;   // [tokens][top], or null: the router has no such outputs
+  const float* wt;  // [tokens][top]
+  const void* h;    // [tokens][W] rows h_stride apart, in the model's precision
+  int h_stride, experts;
+};
+
 // out[t][c] = (base ? base[t][c] : 0) + sum_k parts[t][k][c], in a fixed order; with ``zgate`` (32-bit, z_stride words from
 // token to token) the base is multiplied by sigmoid(zgate[t])
 template <typename T>
 __global__ void moe_combine_kernel(T* __restrict__ out, const T* __restrict__ base, const float* __restrict__ zgate, int z_stride,
-                                   const float* __restrict__ parts, int top, int W, size_t count) {
+                                   const float* __restrict__ parts, const MoeIdentity id, int top, int W, size_t count) {
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < count; i += (size_t)gridDim.x * blockDim.x) {
     const size_t t = i / W, c = i % W;
     float acc = 0.f;
-    for (int k = 0; k < top; ++k) acc += parts[(t * top + k) * W + c];
+    for (int k = 0; k < top; ++k) {
+      if (id.sel && id.sel[t * top + k] >= id.experts)
+        acc = fmaf(id.wt[t * top + k], to_f(((const T*)id.h)[t * id.h_stride + c]), acc);
+      else
+        acc += parts[(t * top + k) * W + c];
+    }
     if (base) acc += to_f(base[i]) * (zgate ? 1.f / (1.f + expf(-zgate[t * z_stride])) : 1.f);
     out[i] = from_f<T>(acc);
   }
 }
 
-extern "C" int ns_moe_combine(void* out, const void* base, const float* zgate, int z_stride, const float* parts, int n, int top, int W, int dtype, hipStream_t stream) {
-  if (n <= 0 || top <= 0 || W <= 0) return NS_ERR_BAD_ARG;
+extern "C" int ns_moe_combine(void* out, const void* base, const float* zgate, int z_stride, const float* parts, const int* sel, const float* wt,
+                              const void* h, int h_stride, int experts, int n, int top, int W, int dtype, hipStream_t stream) {
+  if (n <= 0 || top <= 0 || W <= 0 || (sel && (!wt || !h || experts <= 0))) return NS_ERR_BAD_ARG;
+  const MoeIdentity id{sel, wt, h, h_stride, experts};
   const size_t count = (size_t)n * W;
   size_t blocks = (count + 255) / 256;
   if (blocks > 65535) blocks = 65535;
   if (dtype == NS_DTYPE_F32)
-    moe_combine_kernel<float><<<(int)blocks, 256, 0, stream>>>((float*)out, (const float*)base, zgate, z_stride, parts, top, W, count);
+    moe_combine_kernel<float><<<(int)blocks, 256, 0, stream>>>((float*)out, (const float*)base, zgate, z_stride, parts, id, top, W, count);
   else if (dtype == NS_DTYPE_BF16)
-    moe_combine_kernel<bf16_t><<<(int)blocks, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)base, zgate, z_stride, parts, top, W, count);
+    moe_combine_kernel<bf16_t><<<(int)blocks, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)base, zgate, z_stride, parts, id, top, W, count);
   else
     return NS_ERR_UNSUPPORTED;
   return ns_launch_status();
@@ -596,6 +628,39 @@ extern "C" int ns_scaled_sum(void* out, const void* a, const void* b, const void
     scaled_sum_kernel<float><<<(int)blocks, 256, 0, stream>>>((float*)out, (const float*)a, (const float*)b, (const float*)bias, (const float*)bias_b, sa, sb, W, count);
   else if (dtype == NS_DTYPE_BF16)
     scaled_sum_kernel<bf16_t><<<(int)blocks, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)a, (const bf16_t*)b, (const bf16_t*)bias, (const bf16_t*)bias_b, sa, sb, W, count);
+  else
+    return NS_ERR_UNSUPPORTED;
+  return ns_launch_status();
+}
+
+// The same with a norm behind each side: out = sa * rms(a + bias_a) * wa + sb * rms(b + bias_b) * wb, rms over the row, in 32-bit.
+// One workgroup a row.
+template <typename T>
+__global__ __launch_bounds__(256) void normed_sum_kernel(T* __restrict__ out, const T* __restrict__ a, const T* __restrict__ b,
+                                                         const T* __restrict__ bias, const T* __restrict__ bias_b, const T* __restrict__ wa,
+                                                         const T* __restrict__ wb, float sa, float sb, int W, float eps) {
+  __shared__ float scratch[16];
+  const size_t at = (size_t)blockIdx.x * W;
+  float ssa = 0.f, ssb = 0.f;
+  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+    const float av = to_f(a[at + c]) + (bias ? to_f(bias[c]) : 0.f), bv = to_f(b[at + c]) + (bias_b ? to_f(bias_b[c]) : 0.f);
+    ssa = fmaf(av, av, ssa), ssb = fmaf(bv, bv, ssb);
+  }
+  const float fa = sa / sqrtf(block_sum(ssa, scratch) / (float)W + eps);
+  const float fb = sb / sqrtf(block_sum(ssb, scratch) / (float)W + eps);
+  for (int c = threadIdx.x; c < W; c += blockDim.x) {
+    const float av = to_f(a[at + c]) + (bias ? to_f(bias[c]) : 0.f), bv = to_f(b[at + c]) + (bias_b ? to_f(bias_b[c]) : 0.f);
+    out[at + c] = from_f<T>(av * fa * to_f(wa[c]) + bv * fb * to_f(wb[c]));
+  }
+}
+
+extern "C" int ns_normed_sum(void* out, const void* a, const void* b, const void* bias, const void* bias_b, const void* wa, const void* wb, float sa,
+                             float sb, int n, int W, float eps, int dtype, hipStream_t stream) {
+  if (n <= 0 || W <= 0 || !wa || !wb) return NS_ERR_BAD_ARG;
+  if (dtype == NS_DTYPE_F32)
+    normed_sum_kernel<float><<<n, 256, 0, stream>>>((float*)out, (const float*)a, (const float*)b, (const float*)bias, (const float*)bias_b, (const float*)wa, (const float*)wb, sa, sb, W, eps);
+  else if (dtype == NS_DTYPE_BF16)
+    normed_sum_kernel<bf16_t><<<n, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)a, (const bf16_t*)b, (const bf16_t*)bias, (const bf16_t*)bias_b, (const bf16_t*)wa, (const bf16_t*)wb, sa, sb, W, eps);
   else
     return NS_ERR_UNSUPPORTED;
   return ns_launch_status();

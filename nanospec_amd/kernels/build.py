@@ -28,7 +28,7 @@ ARCH = "gfx950"
 FLAGS = ["-O3", "-std=c++17", "-fPIC", "-shared", f"--offload-arch={ARCH}",
          "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-Wno-unused-command-line-argument"]
 
-CORE_SOURCES = ["elementwise.hip", "gemm_generic.hip", "attn_generic.hip", "sampling.hip", "gemm_bf16.hip", "gemm_wide.hip", "graph.hip", "streams.hip", "delta.hip", "latent.hip", "memory.hip", "moe.hip", "retention.hip"]
+CORE_SOURCES = ["elementwise.hip", "gemm_generic.hip", "attn_generic.hip", "sampling.hip", "gemm_bf16.hip", "gemm_wide.hip", "graph.hip", "streams.hip", "delta.hip", "latent.hip", "memory.hip", "moe.hip", "retention.hip", "mamba.hip"]
 ATTN_SOURCES = ["attn_mfma.hip"]
 WIDE_SOURCES = ["attn_wide.hip"]
 

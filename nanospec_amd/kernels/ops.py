@@ -1209,87 +1209,215 @@ def retention_prep(proj: torch.Tensor, offsets: tuple[int, int, int], positions,
     return out
 
 
-RETENTION_MAX_KEY_DIM = 512  # key channels of a head that ``retention_scan`` takes (a column's channels are 8 to a lane of one wave)
+RETENTION_MAX_KEY_DIM = 512  # key channels of a head that ``decay_scan`` takes (a column's channels are 8 to a lane of one wave)
 
 
-RETENTION_CHUNK = 64  # tokens of a chunk in ``retention_chunks``
+RETENTION_CHUNK = 64  # tokens of a chunk in ``decay_chunks``
 RETENTION_CHUNK_INTS = 4  # ints that describe one
 
 
+class DecayRows:
+    """Where a decayed recurrence (``decay_scan``, ``decay_chunks``) finds its operands.  ``rows`` float32 [tokens, width]:
+    q and k of ``kv_heads`` heads of ``key_dim`` channels and v of ``heads`` heads of ``value_dim`` at the columns ``offsets`` (q,
+    k, v); head h reads q and k of head h // (heads / kv_heads).  Exactly one of: ``decay`` float32 [heads] (fixed per head);
+    ``log_decay`` float32 [tokens, heads] or [tokens, heads * key_dim] (logarithms, at most 0, per token and head or per token
+    and key channel).  With a decay per token and head, ``value_scale`` float32 [tokens, heads] multiplies a token's k v^T
+    and ``skip`` float32 [heads] adds skip_h v_t to its read-out."""
+
+    def __init__(self, rows: torch.Tensor, offsets: tuple[int, int, int], heads: int, key_dim: int, value_dim: int, kv_heads: int | None = None,
+                 decay: torch.Tensor | None = None, log_decay: torch.Tensor | None = None, value_scale: torch.Tensor | None = None,
+                 skip: torch.Tensor | None = None) -> None:
+        G = heads if kv_heads is None else kv_heads
+        _f32(rows, "rows")
+        n = rows.shape[0]
+        for t, name in ((decay, "decay"), (log_decay, "log_decay"), (value_scale, "value_scale"), (skip, "skip")):
+            if t is not None:
+                _f32(t, name)
+        q, k, v = offsets
+        if (rows.dim() != 2 or heads <= 0 or G <= 0 or heads % G or min(offsets) < 0 or max(q, k) + G * key_dim > rows.shape[1]
+                or v + heads * value_dim > rows.shape[1]):
+            raise KernelRefused(f"a decayed recurrence of {heads} heads of {key_dim} x {value_dim} over {G}: the row does not hold its operands")
+        if (decay is None) == (log_decay is None) or (decay is not None and decay.numel() != heads):
+            raise KernelRefused("a decayed recurrence has a decay per head, or the logarithms of a decay per token")
+        if decay is not None:
+            self.kind = 0
+        elif log_decay.shape == (n, heads):
+            self.kind = 1
+        elif log_decay.shape == (n, heads * key_dim):
+            self.kind = 2
+        else:
+            raise KernelRefused(f"the logarithms of the decays are [{n}, {heads}] or [{n}, {heads * key_dim}]")
+        if (value_scale is not None or skip is not None) and self.kind != 1:
+            raise KernelRefused("weights of k v^T and a skip go with a decay per token and head")
+        if (value_scale is not None and value_scale.shape != (n, heads)) or (skip is not None and skip.numel() != heads):
+            raise KernelRefused(f"weights of k v^T are [{n}, {heads}], a skip is [{heads}]")
+        self.rows, self.offsets, self.heads, self.kv_heads, self.key_dim, self.value_dim = rows, offsets, heads, G, key_dim, value_dim
+        self.decay, self.log_decay, self.value_scale, self.skip = decay, log_decay, value_scale, skip
+
+    @property
+    def words(self) -> int:
+        """32-bit words of a request's state, [heads, value_dim, key_dim]."""
+        return self.heads * self.value_dim * self.key_dim
+
+    def args(self):
+        return (_ptr(self.rows), c_int(self.rows.shape[1]), *(c_int(o) for o in self.offsets), _ptr(self.decay), _ptr(self.log_decay),
+                _ptr(self.value_scale), _ptr(self.skip), c_int(self.kind))
+
+    def sizes(self):
+        return c_int(self.heads), c_int(self.kv_heads), c_int(self.key_dim), c_int(self.value_dim)
+
+    def state_stride(self, state: torch.Tensor, what: str) -> int:
+        if state.dtype != torch.float32 or state.dim() != 2 or not state.is_contiguous() or not state.is_cuda or state.shape[1] < self.words:
+            raise KernelRefused(f"{what}: the state is float32 [slots, >= {self.words}] on the GPU")
+        return state.shape[1]
+
+
+def decay_chunks_take(key_dim: int, row_width: int, offsets: tuple[int, int, int]) -> bool:
+    """Whether ``decay_chunks`` takes these sizes: a lane reads four neighbouring key channels at a time."""
+    return key_dim % 4 == 0 and row_width % 4 == 0 and offsets[0] % 4 == 0 and offsets[1] % 4 == 0
+
+
 def retention_chunks_take(heads: int, key_dim: int, value_dim: int) -> bool:
-    """Whether ``retention_chunks`` takes these sizes: a lane reads four neighbouring key channels at a time."""
-    return key_dim % 4 == 0 and (heads * (2 * key_dim + value_dim)) % 4 == 0
+    """The same for rows [q | k | v] as ``retention_prep`` leaves them."""
+    return decay_chunks_take(key_dim, heads * (2 * key_dim + value_dim), (0, heads * key_dim, 2 * heads * key_dim))
+
+
+def decay_chunks(r: DecayRows, state: torch.Tensor, chunks: torch.Tensor, state_slots, workspace: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """``decay_scan`` for the requests that ``chunks`` cuts into chunks of up to ``RETENTION_CHUNK`` tokens (all but a
+    request's last one full), in 32-bit matrix products.  ``chunks`` int32 [n, RETENTION_CHUNK_INTS]: request, row of the first
+    token, tokens (0: describes nothing), and, for a request's first chunk, how many follow one another from it (else 0);
+    ``workspace`` float32 [n * heads * value_dim * key_dim].  ``r.log_decay`` is left holding sums in the rows of the chunks."""
+    _f32(out, "out"), _f32(workspace, "workspace"), _i32(chunks, "chunks"), _i32(state_slots, "state_slots")
+    _gpu(chunks, state_slots)
+    stride = r.state_stride(state, "decay_chunks")
+    if (not decay_chunks_take(r.key_dim, r.rows.shape[1], r.offsets) or out.shape != (r.rows.shape[0], r.heads * r.value_dim) or stride % 4
+            or chunks.dim() != 2 or chunks.shape[1] != RETENTION_CHUNK_INTS or workspace.numel() < chunks.shape[0] * r.words):
+        raise KernelRefused(f"decay_chunks: operands do not fit {r.heads} heads of {r.key_dim} x {r.value_dim} (key sizes in multiples of four)")
+    _check(build.core().ns_retention_chunks(*r.args(), _ptr(state), ctypes.c_longlong(stride), _ptr(chunks), c_int(chunks.shape[0]), _ptr(state_slots),
+                                            _ptr(workspace), _ptr(out), *r.sizes(), _stream()), "decay_chunks")
+    return out
+
+
+def decay_scan(r: DecayRows, state: torch.Tensor, qo_indptr, state_slots, out: torch.Tensor, skip_from: int = 0) -> torch.Tensor:
+    """S <- decay S + k v^T and out = S^T q per head over every request's tokens of the step in order.  ``state`` float32
+    [slots, >= heads * value_dim * key_dim], a request's S as [heads, value_dim, key_dim] in its slot; ``out`` float32 [tokens,
+    heads * value_dim].  ``skip_from`` > 0: requests that bring at least so many tokens are left alone."""
+    _f32(out, "out"), _i32(qo_indptr, "qo_indptr"), _i32(state_slots, "state_slots")
+    _gpu(qo_indptr, state_slots)
+    stride = r.state_stride(state, "decay_scan")
+    if (r.key_dim > RETENTION_MAX_KEY_DIM or out.shape != (r.rows.shape[0], r.heads * r.value_dim) or qo_indptr.numel() != state_slots.numel() + 1):
+        raise KernelRefused(f"decay_scan: operands do not fit {r.heads} heads of {r.key_dim} x {r.value_dim} (key sizes up to {RETENTION_MAX_KEY_DIM})")
+    _check(build.core().ns_retention_scan(*r.args(), _ptr(state), ctypes.c_longlong(stride), _ptr(qo_indptr), _ptr(state_slots), _ptr(out),
+                                          c_int(state_slots.numel()), *r.sizes(), c_int(skip_from), _stream()), "decay_scan")
+    return out
+
+
+def retention_rows(qkv: torch.Tensor, decay: torch.Tensor, heads: int, key_dim: int, value_dim: int) -> DecayRows:
+    """Rows [q | k | v] float32 [tokens, heads * (2 key_dim + value_dim)] as ``retention_prep`` leaves them, one fixed ``decay`` per head."""
+    if qkv.dim() != 2 or qkv.shape[1] != heads * (2 * key_dim + value_dim):
+        raise KernelRefused(f"retention: rows of {heads} heads hold {heads * (2 * key_dim + value_dim)} columns")
+    return DecayRows(qkv, (0, heads * key_dim, 2 * heads * key_dim), heads, key_dim, value_dim, decay=decay)
 
 
 def retention_chunks(qkv: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, chunks: torch.Tensor, state_slots, heads: int, key_dim: int,
                      value_dim: int, workspace: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
-    """``retention_scan`` for the requests that ``chunks`` cuts into chunks of up to ``RETENTION_CHUNK`` tokens (all but a
-    request's last one full), in 32-bit matrix products.  ``chunks`` int32 [n, RETENTION_CHUNK_INTS]: request, row of the first
-    token, tokens (0: describes nothing), and, for a request's first chunk, how many follow one another from it (else 0);
-    ``workspace`` float32 [n * heads * value_dim * key_dim]."""
-    _f32(qkv, "qkv"), _f32(decay, "decay"), _f32(out, "out"), _f32(workspace, "workspace"), _i32(chunks, "chunks"), _i32(state_slots, "state_slots")
-    if state.dtype != torch.float32 or state.dim() != 2 or not state.is_contiguous() or not state.is_cuda:
-        raise KernelRefused("retention_chunks: the state is float32 [slots, floats per slot] on the GPU")
-    n, stride = qkv.shape[0], state.shape[1]
-    words = heads * key_dim * value_dim
-    if (not retention_chunks_take(heads, key_dim, value_dim) or qkv.shape != (n, heads * (2 * key_dim + value_dim)) or decay.numel() != heads
-            or out.shape != (n, heads * value_dim) or stride < words or stride % 4 or chunks.dim() != 2 or chunks.shape[1] != RETENTION_CHUNK_INTS
-            or workspace.numel() < chunks.shape[0] * words):
-        raise KernelRefused(f"retention_chunks: operands do not fit {heads} heads of {key_dim} x {value_dim} (key sizes in multiples of four)")
-    _check(build.core().ns_retention_chunks(_ptr(qkv), _ptr(decay), _ptr(state), ctypes.c_longlong(stride), _ptr(chunks), c_int(chunks.shape[0]),
-                                            _ptr(state_slots), _ptr(workspace), _ptr(out), c_int(heads), c_int(key_dim), c_int(value_dim), _stream()),
-           "retention_chunks")
-    return out
+    """``decay_chunks`` over ``retention_rows``."""
+    return decay_chunks(retention_rows(qkv, decay, heads, key_dim, value_dim), state, chunks, state_slots, workspace, out)
 
 
 def retention_scan(qkv: torch.Tensor, decay: torch.Tensor, state: torch.Tensor, qo_indptr, state_slots, heads: int, key_dim: int, value_dim: int,
                    out: torch.Tensor, skip_from: int = 0) -> torch.Tensor:
-    """S <- decay_h S + k v^T and out = S^T q per head over every request's tokens of the step in order.  ``qkv`` float32
-    [tokens, heads * (2 key_dim + value_dim)] as ``retention_prep`` leaves it; ``decay`` float32 [heads]; ``state`` float32
-    [slots, >= heads * value_dim * key_dim], a request's S as [heads, value_dim, key_dim] in its slot; ``out`` float32 [tokens,
-    heads * value_dim].  ``skip_from`` > 0: requests that bring at least so many tokens are left alone."""
-    _f32(qkv, "qkv"), _f32(decay, "decay"), _f32(out, "out"), _i32(qo_indptr, "qo_indptr"), _i32(state_slots, "state_slots")
-    if state.dtype != torch.float32 or state.dim() != 2 or not state.is_contiguous() or not state.is_cuda:
-        raise KernelRefused("retention_scan: the state is float32 [slots, floats per slot] on the GPU")
-    stride = state.shape[1]
-    n = qkv.shape[0]
-    if (key_dim > RETENTION_MAX_KEY_DIM or qkv.shape != (n, heads * (2 * key_dim + value_dim)) or decay.numel() != heads or out.shape != (n, heads * value_dim)
-            or stride < heads * key_dim * value_dim or qo_indptr.numel() != state_slots.numel() + 1):
-        raise KernelRefused(f"retention_scan: operands do not fit {heads} heads of {key_dim} x {value_dim} (key sizes up to {RETENTION_MAX_KEY_DIM})")
-    _check(build.core().ns_retention_scan(_ptr(qkv), _ptr(decay), _ptr(state), ctypes.c_longlong(stride), _ptr(qo_indptr), _ptr(state_slots), _ptr(out),
-                                          c_int(state_slots.numel()), c_int(heads), c_int(key_dim), c_int(value_dim), c_int(skip_from), _stream()),
-           "retention_scan")
+    """``decay_scan`` over ``retention_rows``."""
+    return decay_scan(retention_rows(qkv, decay, heads, key_dim, value_dim), state, qo_indptr, state_slots, out, skip_from)
+
+
+def log_decay_heads(z: torch.Tensor, bias: torch.Tensor, a_log: torch.Tensor, dt: torch.Tensor, log_decay: torch.Tensor) -> None:
+    """dt[t, h] = softplus(z[t, h] + bias[h]); log_decay[t, h] = -exp(a_log[h]) dt[t, h]: ``z`` [tokens, heads] (may be a column
+    slice) in the model's dtype, everything else float32."""
+    _gpu(z), _f32(bias, "bias"), _f32(a_log, "a_log"), _f32(dt, "dt"), _f32(log_decay, "log_decay")
+    n, heads = dt.shape
+    if z.shape != (n, heads) or z.stride(1) != 1 or log_decay.shape != (n, heads) or bias.numel() != heads or a_log.numel() != heads:
+        raise KernelRefused("log_decay_heads: z, dt and log_decay [tokens, heads], bias and a_log [heads]")
+    _check(build.core().ns_log_decay_heads(_ptr(dt), _ptr(log_decay), _ptr(z), c_int(z.stride(0)), _ptr(bias), _ptr(a_log), c_int(n), c_int(heads),
+                                           c_int(_dtype_code(z)), _stream()), "log_decay_heads")
+
+
+def log_decay_channels(z: torch.Tensor, bias: torch.Tensor, tau: float, log_decay: torch.Tensor) -> torch.Tensor:
+    """log_decay[t, i] = log(sigmoid(z[t, i] + bias[i])) / tau: ``z`` [tokens, width] (may be a column slice) in the model's
+    dtype, everything else float32."""
+    _gpu(z), _f32(bias, "bias"), _f32(log_decay, "log_decay")
+    n, width = log_decay.shape
+    if z.shape != (n, width) or z.stride(1) != 1 or bias.numel() != width or not tau > 0:
+        raise KernelRefused("log_decay_channels: z and log_decay [tokens, width], bias [width], a positive tau")
+    _check(build.core().ns_log_decay_channels(_ptr(log_decay), _ptr(z), c_int(z.stride(0)), _ptr(bias), c_float(1.0 / tau), c_int(n), c_int(width),
+                                              c_int(_dtype_code(z)), _stream()), "log_decay_channels")
+    return log_decay
+
+
+SELECTIVE_SCAN_MAX_STATE = 512
+
+
+def selective_scan(x: torch.Tensor, zdt: torch.Tensor, bc: torch.Tensor, b_off: int, c_off: int, z: torch.Tensor, dt_bias: torch.Tensor,
+                   A: torch.Tensor, skip: torch.Tensor, state: torch.Tensor, qo_indptr, state_slots, out: torch.Tensor) -> torch.Tensor:
+    """Mamba's selective scan over every request's tokens of the step in order (``csrc/mamba.hip``): dt = softplus(zdt + dt_bias);
+    S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n; y_c = sum_n S[c, n] C_n + skip_c x_c; out = y silu(z).  ``x`` float32
+    [tokens, inner]; ``zdt``, ``z`` [tokens, inner] (may be column slices) and ``bc`` (B at the column ``b_off``, C at ``c_off``) in
+    the model's dtype, as ``out``; ``A`` float32 [inner, N]; ``state`` float32 [slots, >= inner * N], [inner, N] in a slot."""
+    _gpu(zdt, bc, z, out, qo_indptr, state_slots)
+    _f32(x, "x"), _f32(dt_bias, "dt_bias"), _f32(A, "A"), _f32(skip, "skip"), _i32(qo_indptr, "qo_indptr"), _i32(state_slots, "state_slots")
+    n, inner = x.shape
+    N = A.shape[1]
+    if (A.shape != (inner, N) or N > SELECTIVE_SCAN_MAX_STATE or dt_bias.numel() != inner or skip.numel() != inner
+            or any(t.shape != (n, inner) or t.stride(1) != 1 for t in (zdt, z, out)) or not out.is_contiguous() or bc.dim() != 2 or bc.shape[0] != n
+            or bc.stride(1) != 1 or min(b_off, c_off) < 0 or max(b_off, c_off) + N > bc.shape[1] or any(t.dtype != out.dtype for t in (zdt, bc, z))
+            or qo_indptr.numel() != state_slots.numel() + 1):
+        raise KernelRefused(f"selective_scan: operands do not fit {inner} channels of {N} states (up to {SELECTIVE_SCAN_MAX_STATE})")
+    if state.dtype != torch.float32 or state.dim() != 2 or not state.is_contiguous() or not state.is_cuda or state.shape[1] < inner * N:
+        raise KernelRefused(f"selective_scan: the state is float32 [slots, >= {inner * N}] on the GPU")
+    _check(build.core().ns_selective_scan(_ptr(x), _ptr(zdt), c_int(zdt.stride(0)), _ptr(bc), c_int(bc.stride(0)), c_int(b_off), c_int(c_off), _ptr(z),
+                                          c_int(z.stride(0)), _ptr(dt_bias), _ptr(A), _ptr(skip), _ptr(state), ctypes.c_longlong(state.shape[1]),
+                                          _ptr(qo_indptr), _ptr(state_slots), _ptr(out), c_int(state_slots.numel()), c_int(inner), c_int(N),
+                                          c_int(_dtype_code(out)), _stream()), "selective_scan")
     return out
 
 
 def gate_mul(x: torch.Tensor, gate: torch.Tensor, out: torch.Tensor, silu: bool = False) -> torch.Tensor:
-    """out = x * sigmoid(gate), or x * gate * sigmoid(gate) with ``silu``, the gate formed in 32-bit; ``gate`` may be a column
-    slice of wider rows; ``x`` and ``out`` contiguous [tokens, width] (they may be one tensor)."""
+    """out = x * sigmoid(gate), or x * gate * sigmoid(gate) with ``silu``, the gate formed in 32-bit; ``gate`` [tokens, width], or
+    [tokens, heads] with width a multiple of heads (a head's channels share its gate), may be a column slice of wider rows;
+    ``x`` and ``out`` contiguous [tokens, width] (they may be one tensor)."""
     _gpu(x, gate, out)
     n, width = x.shape
-    if (not x.is_contiguous() or out.shape != x.shape or not out.is_contiguous() or out.dtype != x.dtype or gate.dtype != x.dtype or gate.shape != x.shape
-            or gate.stride(1) != 1):
-        raise KernelRefused("gate_mul: x and out contiguous [tokens, width], gate [tokens, width] of the same dtype")
-    _check(build.core().ns_gate_mul(_ptr(out), _ptr(x), _ptr(gate), c_int(gate.stride(0)), c_int(n), c_int(width), c_int(1 if silu else 0),
-                                    c_int(_dtype_code(x)), _stream()), "gate_mul")
+    if (not x.is_contiguous() or out.shape != x.shape or not out.is_contiguous() or out.dtype != x.dtype or gate.dtype != x.dtype
+            or gate.dim() != 2 or gate.shape[0] != n or not gate.shape[1] or width % gate.shape[1] or gate.stride(1) != 1):
+        raise KernelRefused("gate_mul: x and out contiguous [tokens, width], gate [tokens, width] or [tokens, heads] of the same dtype")
+    _check(build.core().ns_gate_mul(_ptr(out), _ptr(x), _ptr(gate), c_int(gate.stride(0)), c_int(n), c_int(width), c_int(width // gate.shape[1]),
+                                    c_int(1 if silu else 0), c_int(_dtype_code(x)), _stream()), "gate_mul")
     return out
+
+
+MOE_SCORES = {"softmax": 0, "sigmoid": 1, "softmax_all": 2}  # (numbered as csrc/moe.hip does)
 
 
 def moe_route(h: torch.Tensor, router: torch.Tensor, bias: torch.Tensor | None, top: int, sel: torch.Tensor, weights: torch.Tensor,
               logits: torch.Tensor | None = None, sigmoid: bool = False, correction: torch.Tensor | None = None, groups: int = 1,
-              keep: int = 1, extra: int = 0) -> None:
+              keep: int = 1, extra: int = 0, score: str = "softmax", group_best: int = 2, scale: float = 1.0) -> None:
     """Router logits z = router h + bias in 32-bit (``router`` float32 [experts, W]); ``sel`` int32 [tokens, top] receives the
     experts with the largest logits in falling order, ``weights`` float32 [tokens, top] the soft-max over those logits.
     ``logits``: float32 [tokens, experts], receives z (scratch if the caller has no use for it).
-    ``sigmoid``: the scores are s = sigmoid(z), the choice goes by s + ``correction`` (float32 [experts] or None) and the
-    weights are the chosen s themselves.  ``groups`` > 1: only experts of the ``keep`` groups (of experts / groups neighbours)
-    with the largest sums of their two best choice scores can be chosen.  ``extra``: the last rows of ``router`` (and of
-    ``bias``) that belong to no expert; their logits are left in ``logits`` [tokens, experts + extra] behind the experts'."""
+    ``score`` = "sigmoid" (or ``sigmoid``): the scores are s = sigmoid(z), the choice goes by s + ``correction`` (float32 [experts] or None) and
+    the weights are the chosen s themselves; "softmax_all": s is the soft-max over all logits and the weights are the chosen s
+    over their sum (+ 1e-20).  All weights are multiplied by ``scale``.  ``groups`` > 1: only experts of the ``keep`` groups (of
+    experts / groups neighbours) with the largest sums of their ``group_best`` (1 or 2) best choice scores can be chosen.
+    ``extra``: the last rows of ``router`` (and of ``bias``) that belong to no expert; their logits are left in ``logits``
+    [tokens, experts + extra] behind the experts'."""
     _gpu(h, router, bias, sel, weights, logits, correction)
     rows = router.shape[0]
     experts = rows - extra
-    if correction is not None and (not sigmoid or _f32(correction, "correction").numel() != experts):
-        raise KernelRefused("moe_route: a correction [experts] belongs to sigmoid scores")
+    score = "sigmoid" if sigmoid else score
+    if score not in MOE_SCORES or group_best not in (1, 2):
+        raise KernelRefused(f"moe_route: score {score!r} (known: {sorted(MOE_SCORES)}), the best 1 or 2 of a group")
+    if correction is not None and (score == "softmax" or _f32(correction, "correction").numel() != experts):
+        raise KernelRefused("moe_route: a correction [experts] belongs to scores, not to logits")
     if extra < 0 or groups < 1 or experts <= 0 or experts % groups or not 1 <= keep <= groups or top > keep * (experts // groups):
         raise KernelRefused(f"moe_route: {experts} experts in {groups} groups of which {keep} are kept, {top} chosen")
     _f32(router, "router"), _f32(weights, "weights"), _i32(sel, "sel")
@@ -1300,8 +1428,8 @@ def moe_route(h: torch.Tensor, router: torch.Tensor, bias: torch.Tensor | None, 
             or (bias is not None and _f32(bias, "bias").numel() != rows) or _f32(logits, "logits").shape != (n, rows) or not logits.is_contiguous()):
         raise KernelRefused("moe_route: h [tokens, W], router [experts, W], bias [experts], sel and weights [tokens, top], logits [tokens, experts]")
     _check(build.core().ns_moe_route(_ptr(h), c_int(h.stride(0)), _ptr(router), _ptr(bias), _ptr(logits), _ptr(sel), _ptr(weights), c_int(n), c_int(W),
-                                     c_int(experts), c_int(extra), c_int(top), c_int(1 if sigmoid else 0), _ptr(correction), c_int(groups), c_int(keep),
-                                     c_int(_dtype_code(h)), _stream()), "moe_route")
+                                     c_int(experts), c_int(extra), c_int(top), c_int(MOE_SCORES[score]), _ptr(correction), c_int(groups), c_int(keep),
+                                     c_int(group_best), c_float(scale), c_int(_dtype_code(h)), _stream()), "moe_route")
 
 
 def _expert_form(gate, up, act: str | None, what: str):
@@ -1320,7 +1448,8 @@ def moe_expert_rows(h: torch.Tensor, gate: torch.Tensor | None, up: torch.Tensor
     """out[t, k] = weights[t, k] * expert sel[t, k] of h[t], for few rows: every (token, chosen expert) streams that expert's
     matrices, cut into slices over many workgroups.  ``gate``, ``up`` [experts, ff, W], ``down`` [experts, W, ff] in the dtype
     of ``h``; ``act`` float32 [tokens, top, ff] (scratch); ``out`` float32 [tokens, top, W].  ``gate`` = None: experts W_down
-    act(W_up h) with the ``activation`` of that name."""
+    act(W_up h) with the ``activation`` of that name.  Pairs whose ``sel`` is not one of the experts are left out: their rows
+    of ``out`` stay as they are (``moe_combine`` with ``identity``)."""
     _gpu(h, gate, up, down, sel, weights, act, out)
     _f32(out, "out"), _f32(act, "act"), _f32(weights, "weights"), _i32(sel, "sel")
     n, W = h.shape
@@ -1332,8 +1461,8 @@ def moe_expert_rows(h: torch.Tensor, gate: torch.Tensor | None, up: torch.Tensor
             or any(t.dtype != h.dtype or not t.is_contiguous() for t in (gate, up, down) if t is not None)):
         raise KernelRefused("moe_expert_rows: gate and up [experts, ff, W], down [experts, W, ff] in the dtype of h; act [tokens, top, ff] and out [tokens, top, W] float32")
     _check(build.core().ns_moe_expert_rows(_ptr(h), c_int(h.stride(0)), _ptr(gate), _ptr(up), _ptr(down), _ptr(sel), _ptr(weights), _ptr(act),
-                                           _ptr(out), c_int(n), c_int(W), c_int(ff), c_int(top), c_float(limit), c_float(alpha), c_float(shift),
-                                           kind, c_int(_dtype_code(h)), _stream()), "moe_expert_rows")
+                                           _ptr(out), c_int(n), c_int(W), c_int(ff), c_int(top), c_int(experts), c_float(limit), c_float(alpha),
+                                           c_float(shift), kind, c_int(_dtype_code(h)), _stream()), "moe_expert_rows")
     return out
 
 
@@ -1394,9 +1523,11 @@ def clipped_glu(gu: torch.Tensor, limit: float, alpha: float, out: torch.Tensor,
     return out
 
 
-def moe_combine(parts: torch.Tensor, base: torch.Tensor | None, out: torch.Tensor, gate: torch.Tensor | None = None) -> torch.Tensor:
+def moe_combine(parts: torch.Tensor, base: torch.Tensor | None, out: torch.Tensor, gate: torch.Tensor | None = None,
+                identity: tuple | None = None) -> torch.Tensor:
     """out[t] = base[t] + sum_k parts[t, k] (``parts`` float32 [tokens, top, W]; ``base`` and ``out`` in the model's dtype).
-    ``gate`` (float32 [tokens], may be a column of wider rows): the base is multiplied by its sigmoid, token by token."""
+    ``gate`` (float32 [tokens], may be a column of wider rows): the base is multiplied by its sigmoid, token by token.
+    ``identity`` = (sel, weights, h, experts): where sel[t, k] >= experts, weights[t, k] * h[t] takes the place of parts[t, k]."""
     _gpu(parts, base, out, gate)
     if gate is not None and (base is None or gate.dtype != torch.float32 or gate.shape != (parts.shape[0],)):
         raise KernelRefused("moe_combine: a gate is float32 [tokens] and belongs to a base")
@@ -1404,8 +1535,15 @@ def moe_combine(parts: torch.Tensor, base: torch.Tensor | None, out: torch.Tenso
     n, top, W = parts.shape
     if out.shape != (n, W) or not out.is_contiguous() or (base is not None and (base.shape != (n, W) or not base.is_contiguous() or base.dtype != out.dtype)):
         raise KernelRefused("moe_combine: base and out are contiguous [tokens, W] of one dtype")
-    _check(build.core().ns_moe_combine(_ptr(out), _ptr(base), _ptr(gate), c_int(gate.stride(0) if gate is not None else 0), _ptr(parts), c_int(n), c_int(top), c_int(W), c_int(_dtype_code(out)), _stream()),
-           "moe_combine")
+    sel, wt, h, experts = identity if identity is not None else (None, None, None, 0)
+    if identity is not None:
+        _gpu(h, sel)
+        if (_i32(sel, "sel").shape != (n, top) or _f32(wt, "weights").shape != (n, top) or h.shape != (n, W) or h.stride(1) != 1 or h.dtype != out.dtype
+                or experts <= 0):
+            raise KernelRefused("moe_combine: identity experts come with sel and weights [tokens, top], the input [tokens, W] and the number of experts")
+    _check(build.core().ns_moe_combine(_ptr(out), _ptr(base), _ptr(gate), c_int(gate.stride(0) if gate is not None else 0), _ptr(parts), _ptr(sel), _ptr(wt),
+                                       _ptr(h), c_int(h.stride(0) if h is not None else 0), c_int(experts), c_int(n), c_int(top), c_int(W),
+                                       c_int(_dtype_code(out)), _stream()), "moe_combine")
     return out
 
 
@@ -1421,6 +1559,21 @@ def scaled_sum(a: torch.Tensor, b: torch.Tensor, sa: float, sb: float, out: torc
             raise KernelRefused("scaled_sum: a bias is [W] of the same dtype")
     _check(build.core().ns_scaled_sum(_ptr(out), _ptr(a), _ptr(b), _ptr(bias), _ptr(bias_b), c_float(sa), c_float(sb), c_int(n), c_int(W),
                                       c_int(_dtype_code(a)), _stream()), "scaled_sum")
+    return out
+
+
+def normed_sum(a: torch.Tensor, b: torch.Tensor, sa: float, sb: float, wa: torch.Tensor, wb: torch.Tensor, eps: float, out: torch.Tensor,
+               bias: torch.Tensor | None = None, bias_b: torch.Tensor | None = None) -> torch.Tensor:
+    """out = sa * rms(a + bias) * wa + sb * rms(b + bias_b) * wb, rms over the row, formed in 32-bit (weights and biases [W])."""
+    _gpu(a, b, out, wa, wb, bias, bias_b)
+    n, W = a.shape
+    if any(t.shape != (n, W) or not t.is_contiguous() or t.dtype != a.dtype for t in (a, b, out)):
+        raise KernelRefused("normed_sum: a, b and out are contiguous [tokens, W] of one dtype")
+    for t in (wa, wb, bias, bias_b):
+        if t is not None and (t.numel() != W or t.dtype != a.dtype or not t.is_contiguous()):
+            raise KernelRefused("normed_sum: a weight or bias is [W] of the same dtype")
+    _check(build.core().ns_normed_sum(_ptr(out), _ptr(a), _ptr(b), _ptr(bias), _ptr(bias_b), _ptr(wa), _ptr(wb), c_float(sa), c_float(sb), c_int(n),
+                                      c_int(W), c_float(eps), c_int(_dtype_code(a)), _stream()), "normed_sum")
     return out
 
 
@@ -1600,11 +1753,12 @@ def _state_args(state: torch.Tensor, what: str):
 
 
 def conv_silu_carry(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, conv_off: int, token_req, qo_indptr, state_slots,
-                    out: torch.Tensor) -> torch.Tensor:
-    """A short causal convolution over time per channel, then SiLU, across steps.  ``x`` [tokens, >= C] (its first C columns
-    are convolved), ``taps`` float32 [C, K] whose last column multiplies the current token; the K - 1 inputs before a
-    request's first token of this step are read from ``state[slot, conv_off:]`` as [K - 1, C] (zeros for a new request)
-    and replaced afterwards by the last K - 1 inputs including this step's.  ``out`` float32 [tokens, C]."""
+                    out: torch.Tensor, bias: torch.Tensor | None = None, copy: torch.Tensor | None = None) -> torch.Tensor:
+    """A short causal convolution over time per channel (plus ``bias`` float32 [C]), then SiLU, across steps.  ``x`` [tokens, >= C]
+    (its first C columns are convolved), ``taps`` float32 [C, K] whose last column multiplies the current token; the K - 1
+    inputs before a request's first token of this step are read from ``state[slot, conv_off:]`` as [K - 1, C] (zeros for a new
+    request) and replaced afterwards by the last K - 1 inputs including this step's.  ``out`` float32 [tokens, C]; ``copy``
+    [tokens, C] receives the same values in the dtype of ``x``."""
     _gpu(x), _f32(taps, "taps"), _f32(out, "out")
     for name, t in (("token_req", token_req), ("qo_indptr", qo_indptr), ("state_slots", state_slots)):
         _i32(t, name)
@@ -1614,9 +1768,13 @@ def conv_silu_carry(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, co
         raise KernelRefused("conv_silu_carry: x is [tokens, >= C], out float32 [tokens, C], qo_indptr [requests + 1]")
     if K > MAX_CONV_TAPS or conv_off + (K - 1) * C > state.shape[1]:
         raise KernelRefused(f"conv_silu_carry: at most {MAX_CONV_TAPS} taps, and the carried inputs must fit the slot")
+    if bias is not None and _f32(bias, "bias").numel() != C:
+        raise KernelRefused(f"conv_silu_carry: a bias is float32 [{C}]")
+    if copy is not None and (not copy.is_cuda or copy.shape != (n, C) or copy.dtype != x.dtype or not copy.is_contiguous()):
+        raise KernelRefused(f"conv_silu_carry: a copy is contiguous [{n}, {C}] in the dtype of x")
     sp, stride = _state_args(state, "conv_silu_carry")
-    _check(build.core().ns_conv_silu_carry(_ptr(out), _ptr(x), c_int(x.stride(0)), _ptr(taps), sp, stride, c_size_t(conv_off), _ptr(token_req),
-                                           _ptr(qo_indptr), _ptr(state_slots), c_int(n), c_int(reqs), c_int(C), c_int(K),
+    _check(build.core().ns_conv_silu_carry(_ptr(out), _ptr(copy), _ptr(x), c_int(x.stride(0)), _ptr(taps), _ptr(bias), sp, stride, c_size_t(conv_off),
+                                           _ptr(token_req), _ptr(qo_indptr), _ptr(state_slots), c_int(n), c_int(reqs), c_int(C), c_int(K),
                                            c_int(_dtype_code(x)), _stream()), "conv_silu_carry")
     return out
 
@@ -1659,11 +1817,12 @@ def delta_scan(qkv: torch.Tensor, g: torch.Tensor, beta: torch.Tensor, state: to
 
 
 def gated_rms(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor | None, eps: float, heads: int, out: torch.Tensor,
-              den: torch.Tensor | None = None, silu: bool = False) -> torch.Tensor:
+              den: torch.Tensor | None = None, silu: bool = False, gate_first: bool = False) -> torch.Tensor:
     """out[t, h, :] = x / sqrt(mean(x^2) + eps) * weight * sigmoid(gate[t, h, :]) with x = o[t, h, :], or o[t, h, :] /
     den[t, h] if ``den`` (float32 [tokens, heads]) is given; ``o`` float32 [tokens, heads * E], ``weight`` float32 [E] (all
     heads share it) or [heads * E] or None (no weight), ``gate`` (may be a column slice) and ``out`` in the model's dtype.
-    ``silu``: the gate is g sigmoid(g) instead of sigmoid(g)."""
+    ``silu``: the gate is g sigmoid(g) instead of sigmoid(g).  ``gate_first``: the gate stands in front of the norm, x = o[t, h, :] *
+    gate and out = x / sqrt(mean(x^2) + eps) * weight."""
     _f32(o, "o")
     if weight is not None:
         _f32(weight, "weight")
@@ -1675,8 +1834,8 @@ def gated_rms(o: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor | None, 
         raise KernelRefused("gated_rms: operands do not fit heads and value size")
     per_head = width // heads if (weight is not None and weight.numel() == width and heads > 1) else 0
     _check(build.core().ns_gated_rms(_ptr(out), _ptr(o), _ptr(gate), c_int(gate.stride(0)), _ptr(weight), c_int(per_head), _ptr(den), c_int(n),
-                                     c_int(heads), c_int(width // heads), c_float(eps), c_int(1 if silu else 0), c_int(_dtype_code(gate)), _stream()),
-           "gated_rms")
+                                     c_int(heads), c_int(width // heads), c_float(eps), c_int(1 if silu else 0), c_int(1 if gate_first else 0), c_int(_dtype_code(gate)),
+                                     _stream()), "gated_rms")
     return out
 
 

@@ -197,12 +197,18 @@ class Attention:
             raise ValueError("biases, whole-projection norms and mixed values belong to a layer with key/value projections of its own")
         if spec.whole_norm_eps is not None and spec.qk_norm_eps is not None:
             raise ValueError("a norm over the whole projection stands alone: no per-head unit norm beside it")
-        if (spec.sink_name or spec.out_gate) and not spec.own_kv:
+        if (spec.sink_name or spec.out_gate or spec.head_gate) and not spec.own_kv:
             raise ValueError("a learned sink and an output gate belong to a layer with key/value projections of its own")
+        if spec.out_gate and spec.head_gate:
+            raise ValueError("the output gate is one number per channel or one per head")
+        self.gate_width = spec.heads * spec.v_dim if spec.out_gate else (spec.heads if spec.head_gate else 0)
         if spec.sink_name and spec.sink:
             raise ValueError("the soft-max has one sink: of score 0, or a learned one")
         self.sink_logits: torch.Tensor | None = None
-        self.head_form = spec.head_norm_eps is not None or spec.value_is_key  # per-head norms with weights, values that are the keys
+        # what one kernel does head by head: per-head norms with weights, values that are the keys, a rotation beside values of
+        # another size than the keys
+        plain_rotation = self.position.rotary_dim > 0 and spec.v_dim != spec.head_dim and spec.whole_norm_eps is None and spec.qk_norm_eps is None
+        self.head_form = spec.head_norm_eps is not None or spec.value_is_key or (plain_rotation and spec.own_kv and not spec.value_mix)
         if self.head_form and (spec.qk_norm_eps is not None or spec.whole_norm_eps is not None or spec.value_mix or not spec.own_kv):
             raise ValueError("per-head norms with weights and values that are the keys stand beside biases and a rotation only")
         if spec.value_is_key and spec.v_dim != spec.head_dim:
@@ -230,7 +236,7 @@ class Attention:
             if not s.value_is_key:
                 out[v] = ((s.kv_heads * s.v_dim, s.hidden), "linear")
         if s.bias:
-            for name in (q, k, v, o):
+            for name in (q, k, v, o) if s.out_bias else (q, k, v):
                 if name in out:
                     out[name + s.bias_suffix] = ((out[name][0][0],), "bias")
         if s.head_norm_eps is not None:
@@ -241,8 +247,8 @@ class Attention:
             out[k + s.whole_norm_suffix] = ((s.kv_heads * s.head_dim,), "norm")
         if s.sink_name:
             out[self.prefix + s.sink_name] = ((s.heads,), "around_zero")
-        if s.out_gate:
-            out[self.prefix + s.gate_name] = ((s.heads * s.v_dim, s.hidden), "linear")
+        if self.gate_width:
+            out[self.prefix + s.gate_name] = ((self.gate_width, s.hidden), "linear")
         if s.value_mix:
             # (a "source" layer's checkpoint holds the tensor too; it is not used there)
             out[self.prefix + s.value_mix_name] = ((), lambda shape, gen: torch.full(shape, 0.5, device=gen.device)
@@ -256,10 +262,12 @@ class Attention:
         rows = s.heads * s.head_dim + (s.kv_heads * (s.head_dim + (0 if s.value_is_key else s.v_dim)) if s.own_kv else 0)
         self.gate_at = rows  # the output gate's logits, if the layer has a gate, are the last columns of the first product
         stacked = (q,) if not s.own_kv else ((q, k) if s.value_is_key else (q, k, v))
-        if s.out_gate:
-            rows += s.heads * s.v_dim
+        if self.gate_width:
+            rows += self.gate_width
             stacked += (self.prefix + s.gate_name,)
-        wqkv = torch.empty((rows, s.hidden), dtype=dtype, device=device)
+        if s.head_gate:  # (a few rows more or less: the product's rows stay aligned)
+            rows = -(-rows // 16) * 16
+        wqkv = (torch.zeros if s.head_gate else torch.empty)((rows, s.hidden), dtype=dtype, device=device)
         at = 0
         for name in stacked:
             t = get(name)
@@ -270,10 +278,11 @@ class Attention:
         self._form = dict(interleaved=bool(getattr(self.position, "interleaved", False)), factor=float(getattr(self.position, "factor", 1.0)))
         to = lambda name: get(name).to(device=device, dtype=dtype).contiguous()
         if s.bias:
-            if s.out_gate:
+            if self.gate_width:
                 raise ValueError("an output gate beside biased projections is not built")
             self.qkv_bias = torch.cat([to(name + s.bias_suffix) for name in stacked]).contiguous()
-            self.out_bias = to(o + s.bias_suffix)
+            if s.out_bias:
+                self.out_bias = to(o + s.bias_suffix)
         if s.head_norm_eps is not None:
             self.q_head_norm, self.k_head_norm = to(q + s.head_norm_suffix), to(k + s.head_norm_suffix)
         if s.whole_norm_eps is not None:
@@ -381,18 +390,19 @@ class Attention:
                                         q_weight=self.q_head_norm, k_weight=self.k_head_norm, value_is_key=s.value_is_key, **self._form)
         elif s.whole_norm_eps is not None and pos.rotary_dim:
             # a norm over the whole of q and of k, then the rotation, then the pages
-            if s.bias or s.value_mix:
-                raise ops.KernelRefused("rotation behind a whole-projection norm together with biases or mixed values is not built")
+            if s.value_mix:
+                raise ops.KernelRefused("rotation behind a whole-projection norm together with mixed values is not built")
             ops.whole_norm_kv_write(qkv, ctx.positions, ctx.token_req, table, cache.k, cache.v, s.heads, s.kv_heads, s.head_dim, s.v_dim,
-                                    s.whole_norm_eps, q_weight=self.q_norm, k_weight=self.k_norm, inv_freq=pos.inv_freq,
+                                    s.whole_norm_eps, bias=self.qkv_bias, q_weight=self.q_norm, k_weight=self.k_norm, inv_freq=pos.inv_freq,
                                     rotary_dim=pos.rotary_dim, **self._form)
         elif pos.rotary_dim:
             if s.qk_norm_eps is not None or s.v_dim != s.head_dim or not s.own_kv:
                 raise ops.KernelRefused("rotation together with unit-RMS queries and keys, another value size or borrowed keys is not built")
             if s.bias or s.value_mix:
                 raise ops.KernelRefused("rotation together with biases or mixed values is not built")
-            ops.rope_kv_write(qkv, ctx.positions, ctx.token_req, table, pos.inv_freq, cache.k, cache.v, s.heads, s.kv_heads,
-                              s.head_dim, pos.rotary_dim, write_kv=True, **self._form)
+            # (a gate's logits stand behind q, k and v in the row)
+            ops.rope_kv_write(qkv[:, : (s.heads + 2 * s.kv_heads) * s.head_dim], ctx.positions, ctx.token_req, table, pos.inv_freq, cache.k, cache.v,
+                              s.heads, s.kv_heads, s.head_dim, pos.rotary_dim, write_kv=True, **self._form)
         elif s.bias or s.whole_norm_eps is not None or s.value_mix:
             if s.qk_norm_eps is not None:
                 raise ops.KernelRefused("a per-head unit norm together with biases, a whole-projection norm or mixed values is not built")
@@ -421,8 +431,8 @@ class Attention:
             ops.attention_generic(qkv, att, cache.k, cache.v, ctx.token_req, ctx.positions, table, s.heads, s.kv_heads, s.head_dim,
                                   s.softmax_scale, window=s.window, v_dim=s.v_dim, chunk=s.chunk, cap=s.score_cap, sink=s.sink,
                                   slope_exp=s.slope_exp, sink_logits=self.sink_logits)
-        if s.out_gate:
-            ops.gate_mul(att, qkv[:, self.gate_at : self.gate_at + s.heads * s.v_dim], out=att)
+        if self.gate_width:
+            ops.gate_mul(att, qkv[:, self.gate_at : self.gate_at + self.gate_width], out=att)
         if residual is not None and self.out_bias is None:
             return self.wo.into_residual(att, residual, arena=ctx.arena, plain_copy=not ctx.captured)
         y = self.wo(att, out=out if out is not None else ctx.arena.take((n, s.hidden), x.dtype), arena=ctx.arena, plain_copy=not ctx.captured)

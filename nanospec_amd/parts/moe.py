@@ -4,6 +4,9 @@
   the ``top`` largest logits are chosen; their weights are the soft-max over the chosen logits alone
   (``score`` = "sigmoid": s = sigmoid(z); the choice goes by s + correction, inside the ``keep_groups`` groups of neighbouring
   experts whose two largest choice scores add up highest; the weights are the chosen s, not renormalized)
+  (``score`` = "softmax_all": s = soft-max over all logits, the choice likewise by s + correction, the weights are the chosen s
+  over their sum; a group may be judged by its one largest choice score, ``group_best`` = 1)
+  all weights are multiplied by ``weight_scale``; the last ``identity`` outputs of the router are experts that return their input
   expert(h) = W_down (g sigmoid(alpha g) (u + shift)),  g = min(W_gate h, limit),  u = clamp(W_up h, -limit, limit)
   (limit infinite, alpha 1, shift 0: W_down (silu(W_gate h) * W_up h)); or, without a gate matrix, W_down act(W_up h)
   y = sum over the chosen experts of weight * expert(h)  +  shared(h)
@@ -30,14 +33,17 @@ class MoE:
     takes_layouts = True
 
     def __init__(self, spec, prefix: str) -> None:
-        if not 0 < spec.top <= spec.experts or spec.top > ops.MOE_MAX_TOP or spec.experts > ops.MOE_MAX_EXPERTS:
-            raise ValueError(f"{spec.top} of {spec.experts} experts (at most {ops.MOE_MAX_TOP} of {ops.MOE_MAX_EXPERTS})")
-        if spec.score not in ("softmax", "sigmoid"):
-            raise ValueError(f"score={spec.score!r}: use 'softmax' or 'sigmoid'")
-        if spec.correction_name and spec.score != "sigmoid":
-            raise ValueError("a correction on the choice belongs to sigmoid scores")
-        if spec.groups < 1 or spec.experts % spec.groups or not 1 <= spec.keep_groups <= spec.groups or spec.top > spec.keep_groups * (spec.experts // spec.groups):
-            raise ValueError(f"{spec.experts} experts in {spec.groups} groups of which {spec.keep_groups} are kept, {spec.top} chosen")
+        outputs = spec.experts + spec.identity  # what the router chooses from
+        if not 0 < spec.top <= outputs or spec.top > ops.MOE_MAX_TOP or outputs > ops.MOE_MAX_EXPERTS or spec.experts < 1 or spec.identity < 0:
+            raise ValueError(f"{spec.top} of {outputs} experts (at most {ops.MOE_MAX_TOP} of {ops.MOE_MAX_EXPERTS})")
+        if spec.score not in ops.MOE_SCORES:
+            raise ValueError(f"score={spec.score!r}: use one of {sorted(ops.MOE_SCORES)}")
+        if spec.correction_name and spec.score == "softmax":
+            raise ValueError("a correction on the choice belongs to scores, not to logits")
+        if spec.groups < 1 or outputs % spec.groups or not 1 <= spec.keep_groups <= spec.groups or spec.top > spec.keep_groups * (outputs // spec.groups):
+            raise ValueError(f"{outputs} experts in {spec.groups} groups of which {spec.keep_groups} are kept, {spec.top} chosen")
+        if spec.group_best not in (1, 2):
+            raise ValueError(f"group_best={spec.group_best}: a group is judged by its best or its two best")
         # experts without gate matrices: their activation by name (None: gated experts)
         self.act = spec.expert.activation if isinstance(spec.expert, PlainFFSpec) else None
         if self.act is not None and self.act not in ops.ACTIVATIONS:
@@ -47,6 +53,7 @@ class MoE:
         if spec.shared_gate_name and (spec.shared is None or spec.router_bias_name):
             raise ValueError("a gate on the shared expert goes with a shared expert and a router without a bias")
         self.spec, self.prefix = spec, prefix
+        self.outputs = outputs
 
     def _expert(self, e: int, which: int) -> str:
         return f"{self.prefix}{self.spec.expert_prefix}{e}.{self.spec.names[which]}"
@@ -57,11 +64,11 @@ class MoE:
     def wanted(self) -> dict:
         s = self.spec
         ff = s.expert.intermediate
-        out = {self.prefix + s.router_name: ((s.experts, s.hidden), "linear")}
+        out = {self.prefix + s.router_name: ((self.outputs, s.hidden), "linear")}
         if s.router_bias_name:
-            out[self.prefix + s.router_bias_name] = ((s.experts,), "bias")
+            out[self.prefix + s.router_bias_name] = ((self.outputs,), "bias")
         if s.correction_name:
-            out[self.prefix + s.correction_name] = ((s.experts,), "bias")
+            out[self.prefix + s.correction_name] = ((self.outputs,), "bias")
         for e in range(s.experts):
             if self.act is None:
                 out[self._expert(e, 0)] = ((ff, s.hidden), "linear")
@@ -86,7 +93,7 @@ class MoE:
         if s.shared_gate_name:
             router.append(get(self.prefix + s.shared_prefix + s.shared_gate_name))
         self.router = torch.cat([t.to(device=device, dtype=torch.float32) for t in router]).contiguous()
-        self.extra = self.router.shape[0] - s.experts
+        self.extra = self.router.shape[0] - self.outputs
         f32 = lambda name: get(self.prefix + name).to(device=device, dtype=torch.float32).contiguous() if name else None
         self.router_bias, self.correction = f32(s.router_bias_name), f32(s.correction_name)
         self.shared_in = self.shared_out = None
@@ -99,9 +106,9 @@ class MoE:
         s = self.spec
         n, take = x.shape[0], ctx.arena.take
         sel, wt = take((n, s.top), torch.int32), take((n, s.top), torch.float32)
-        z = take((n, s.experts + self.extra), torch.float32)
-        ops.moe_route(x, self.router, self.router_bias, s.top, sel, wt, logits=z, sigmoid=s.score == "sigmoid", correction=self.correction,
-                      groups=s.groups, keep=s.keep_groups, extra=self.extra)
+        z = take((n, self.outputs + self.extra), torch.float32)
+        ops.moe_route(x, self.router, self.router_bias, s.top, sel, wt, logits=z, score=s.score, correction=self.correction,
+                      groups=s.groups, keep=s.keep_groups, extra=self.extra, group_best=s.group_best, scale=s.weight_scale)
         base = None
         if s.shared is not None:
             sf = s.shared.intermediate
@@ -115,7 +122,8 @@ class MoE:
         form = (e.limit, e.alpha, take, e.shift) if self.act is None else (0.0, 0.0, take, 0.0, self.act)
         parts = ops.moe_experts(x, self.gate, self.up, self.down, sel, wt, *form)
         return ops.moe_combine(parts, base, out if out is not None else take((n, s.hidden), x.dtype),
-                               gate=z[:, s.experts] if s.shared_gate_name else None)
+                               gate=z[:, self.outputs] if s.shared_gate_name else None,
+                               identity=(sel, wt, x, s.experts) if s.identity else None)
 
 
 registry.register("ffn", "moe", MoE)

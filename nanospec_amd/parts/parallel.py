@@ -1,4 +1,5 @@
-"""Two mixers side by side ("parallel"): both read the same input, y = left_scale * left(h) + right_scale * right(h).
+"""Two mixers side by side ("parallel"): both read the same input, y = left_scale * left(h) + right_scale * right(h), or, with a
+norm behind each (``out_norm_eps``), y = left_scale * rms(left(h)) * w_left + right_scale * rms(right(h)) * w_right.
 
 Each of the two is a mixer of any registered kind with its own tensors (under the two prefixes) and its own needs of the
 cache: the pair asks for a tuple of needs and is handed a tuple of views in the same order.  The sum is formed in 32-bit
@@ -21,6 +22,7 @@ class ParallelMixer:
         self.left = registry.build("mixer", spec.left, prefix + spec.prefixes[0])
         self.right = registry.build("mixer", spec.right, prefix + spec.prefixes[1])
         self.sides = (self.left, self.right)
+        self.out_norms: tuple = ()
 
     @property
     def graph_safe(self) -> bool:
@@ -30,6 +32,8 @@ class ParallelMixer:
         out = {}
         for p in self.sides:
             out.update(p.wanted())
+        if self.spec.out_norm_eps is not None:
+            out.update({self.prefix + name: ((self.spec.left.hidden,), "norm") for name in self.spec.out_norm_names})
         return out
 
     def load(self, get, dtype, device, layouts: str = "both") -> None:
@@ -38,6 +42,8 @@ class ParallelMixer:
                 p.load(get, dtype, device, layouts)
             else:
                 p.load(get, dtype, device)
+        if self.spec.out_norm_eps is not None:
+            self.out_norms = tuple(get(self.prefix + name).to(device=device, dtype=dtype).contiguous() for name in self.spec.out_norm_names)
 
     def cache_need(self):
         return tuple(p.cache_need() for p in self.sides)
@@ -68,8 +74,10 @@ class ParallelMixer:
             else:
                 results.append(part.forward(ctx, x, view, owns_cache, out=buf))
             biases.append(bias)
-        return ops.scaled_sum(results[0], results[1], self.spec.left_scale, self.spec.right_scale,
-                              out if out is not None else ctx.arena.take((n, hidden), x.dtype), bias=biases[0], bias_b=biases[1])
+        s, out = self.spec, out if out is not None else ctx.arena.take((n, hidden), x.dtype)
+        if s.out_norm_eps is not None:
+            return ops.normed_sum(*results, s.left_scale, s.right_scale, *self.out_norms, s.out_norm_eps, out, bias=biases[0], bias_b=biases[1])
+        return ops.scaled_sum(*results, s.left_scale, s.right_scale, out, bias=biases[0], bias_b=biases[1])
 
 
 registry.register("mixer", "parallel", ParallelMixer)

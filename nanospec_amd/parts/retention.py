@@ -10,9 +10,9 @@ S lives in 32-bit in the request's state slot and is carried from step to step.
 
 One product reads h for q, k, v and the gate together (the matrices are stacked at load time); rotation and scaling
 (``retention_prep``), the recurrence and the gated norm (``gated_rms``) are 32-bit kernels.  The recurrence takes a
-request's tokens of the step one after the other (``retention_scan``: single tokens, short portions, padding rows, which own
+request's tokens of the step one after the other (``decay_scan``: single tokens, short portions, padding rows, which own
 the pad slot) or, from ``CHUNKED_FROM`` tokens on, in chunks whose tokens meet the state and each other as 32-bit matrix
-products (``retention_chunks``); the two differ by rounding.
+products (``decay_chunks``); the two differ by rounding.
 """
 
 from __future__ import annotations
@@ -31,7 +31,7 @@ CHUNKED_FROM = 192  # a request that brings at least this many tokens runs in ch
 
 
 class ChunkPlan:
-    """The step's long portions as ``ops.retention_chunks`` walks them (a batch plan, see ``engine.context``): every request that
+    """The step's long portions as ``ops.decay_chunks`` walks them (a batch plan, see ``engine.context``): every request that
     brings at least ``CHUNKED_FROM`` tokens cut into chunks.  shape = (chunks, requests left to the scan); a region of a
     fixed shape may hold more chunks than the batch needs: the rest describe nothing."""
 
@@ -67,6 +67,19 @@ class ChunkPlan:
 
 
 CHUNKS = ChunkPlan()
+
+
+def decayed_recurrence(ctx, rows: "ops.DecayRows", state: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """A step's decayed recurrence over the state in the requests' slots: long portions in chunks where the sizes allow it, all
+    other requests by the scan."""
+    takes = ops.decay_chunks_take(rows.key_dim, rows.rows.shape[1], rows.offsets)
+    chunks, rest = ChunkPlan.view(ctx) if takes else (None, 1)
+    # (the scan first: where decays are per token the chunked form leaves sums in their place, in its own rows)
+    if rest:
+        ops.decay_scan(rows, state, ctx.qo_indptr, ctx.state_slots, out, skip_from=CHUNKED_FROM if chunks is not None else 0)
+    if chunks is not None:
+        ops.decay_chunks(rows, state, chunks, ctx.state_slots, ctx.arena.take((chunks.shape[0] * rows.words,), torch.float32), out)
+    return out
 
 
 class Retention:
@@ -139,13 +152,8 @@ class Retention:
         proj = self.w_in(x, out=take((n, self.w_in.n), x.dtype), arena=ctx.arena, plain_copy=not ctx.captured)
         qkv = ops.retention_prep(proj, (0, self.k_at, self.v_at), ctx.positions, pos.inv_freq, s.heads, s.key_dim, s.value_dim, pos.rotary_dim,
                                  s.key_scale, out=take((n, 2 * self.qk + self.vw), torch.float32), silu=s.qkv_silu, **self._form)
-        o = take((n, self.vw), torch.float32)
-        sizes = (s.heads, s.key_dim, s.value_dim)
-        chunks, rest = ChunkPlan.view(ctx) if ops.retention_chunks_take(*sizes) else (None, 1)
-        if chunks is not None:
-            ops.retention_chunks(qkv, self.decay, cache.state, chunks, ctx.state_slots, *sizes, take((chunks.shape[0] * self.qk * s.value_dim,), torch.float32), o)
-        if rest:
-            ops.retention_scan(qkv, self.decay, cache.state, ctx.qo_indptr, ctx.state_slots, *sizes, out=o, skip_from=CHUNKED_FROM if chunks is not None else 0)
+        rows = ops.retention_rows(qkv, self.decay, s.heads, s.key_dim, s.value_dim)
+        o = decayed_recurrence(ctx, rows, cache.state, take((n, self.vw), torch.float32))
         gated = ops.gated_rms(o, proj[:, self.g_at : self.g_at + self.vw], self.norm, s.norm_eps, 1 if s.whole_norm_name else s.heads,
                               out=take((n, self.vw), x.dtype), silu=s.gate_silu)
         return self.w_out(gated, out=out if out is not None else take((n, s.hidden), x.dtype), arena=ctx.arena, plain_copy=not ctx.captured)
