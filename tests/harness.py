@@ -112,3 +112,37 @@ def step_context(lens, starts, tables):
     max_kv = max(s + n for s, n in zip(starts, lens))
     chunk_kv = max((s + n for s, n in zip(starts, lens) if n != 1), default=0)
     return StepContext(layout, torch.from_numpy(host).to(DEV), Arena(DEV), max_position=max_kv - 1, max_kv_len=max_kv, max_chunk_kv=chunk_kv)
+
+
+class PartCtx:
+    """The little that a part asks of a step's context when it is run alone."""
+
+    captured = False
+
+    def __init__(self):
+        from nanospec_amd.engine.arena import Arena
+
+        self.arena, self.plans = Arena(torch.device(DEV)), {}
+
+    def requests(self, lens, slots, positions, plan=None, spare=0):
+        """A batch of hand-made requests; ``plan``: a batch plan that describes it, in a region of ``spare`` more entries than it needs."""
+        import types
+
+        import numpy as np
+
+        self.token_req, self.qo_indptr, self.state_slots = batch(lens, slots)
+        self.positions = torch.tensor(positions, dtype=torch.int32, device=DEV)
+        self.max_position = max(positions)
+        self.plans = {}
+        if plan is not None:
+            shape = plan.shape(lens)
+            shape = (shape[0] + spare, *shape[1:])
+            out = np.full(max(1, plan.ints(shape)), -1, dtype=np.int32)
+            plan.fill(out, shape, types.SimpleNamespace(covered=len(lens), lens=np.array(lens), indptr=np.concatenate([[0], np.cumsum(lens)])))
+            self.plans = {plan.key: (torch.from_numpy(out).to(DEV), shape)}
+
+
+def off(got, want):
+    """The largest difference over the largest value, and the root mean square of the difference over that of the values."""
+    d = got.cpu().double() - want
+    return float(d.abs().max() / want.abs().max()), float(d.pow(2).mean().sqrt() / want.pow(2).mean().sqrt())
