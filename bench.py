@@ -325,16 +325,48 @@ def zipedra_config(shape: dict, layers: int | None = None):
                                   "token_side": {"dim": 256}, "loop": {"start": 1, "stop": 4, "times": 2}, "layers": entries})
 
 
-DESIGNS = {"vuzelix": vuzelix_config, "fetitar": fetitar_config, "padetar": padetar_config, "fimilorn": fimilorn_config, "zipedra": zipedra_config}
-# the existing model that a design is closest to, measured beside it as well (Llama always is): Padetar, like Fimilorn, has a
+# Sizes for ``--design meropel``: the Meropel design at the widths, depths and head counts of the Llama shapes above.  The layers
+# take turns: "parallel" (half the shape's heads and key/value heads with keys of head_dim and values of twice that, a gate per
+# head, beside a selective scan of as many channels as the width with 16 states), "gla" (width / 256 heads of 128 key and 256 value
+# channels), "parallel_2" (the shape's heads and key/value heads, the whole head rotated, beside a Mamba-2 of width / 64 heads of 64
+# channels with 128 states).  The first layer's feed-forward is dense with the shape's inner size; every other is 32 experts of an
+# eighth of it and 4 identity experts in 4 groups of which 2 are kept, four a token, beside a shared expert of half the inner
+# size.  A pair table of 65,536 rows.
+def meropel_config(shape: dict, layers: int | None = None):
+    from dataclasses import replace
+
+    from nanospec_amd.config import MeropelConfig
+
+    n = layers or shape["num_hidden_layers"]
+    heads, kvh, hd, ff, width = (shape["num_attention_heads"], shape["num_key_value_heads"], shape["head_dim"], shape["intermediate_size"],
+                                 shape["hidden_size"])
+    left = dict(heads=heads // 2, kv_heads=kvh // 2, dim=hd, vdim=2 * hd, scale=hd ** -0.5, rot={"base": 1e6, "dims": hd // 2})
+    left_2 = dict(heads=heads, kv_heads=kvh, dim=hd, vdim=hd, scale=hd ** -0.5, rot={"base": 1e6, "dims": hd})
+    mixers = [
+        ("parallel", {"left": left, "right": dict(inner=width, state=16, dt_rank=width // 16, conv=4), "left_scale": 1.0, "right_scale": 1.0}),
+        ("gla", dict(heads=width // 256, dim=128, vdim=256, tau=16.0)),
+        ("parallel_2", {"left": left_2, "right": dict(heads=width // 64, vdim=64, state=128, groups=1, conv=4, norm_groups=1)}),
+    ]
+    moe = {"kind": "moe", "expert": {"ff": ff // 8}, "router": {"experts": 32, "top": 4, "scale": 1.5, "identity": 4, "groups": {"count": 4, "keep": 2}},
+           "shared": {"ff": ff // 2}}
+    entries = [{"type": mixers[i % 3][0], "mixer": mixers[i % 3][1], "mlp": {"kind": "dense", "ff": ff} if i == 0 else moe} for i in range(n)]
+    cfg = MeropelConfig.from_hf({"architecture": "Meropel", "vocab": shape["vocab_size"], "width": width, "norm": {"eps": 1e-6}, "logit_scale": 0.5,
+                                 "embedding": {"bigram": {"buckets": 65536, "mul_prev": 127, "mul_cur": 7}}, "layers": entries})
+    return replace(cfg, layers=tuple(l if l.gla is None else replace(l, gla=replace(l.gla, decay_rank=16)) for l in cfg.layers))
+
+
+DESIGNS = {"vuzelix": vuzelix_config, "fetitar": fetitar_config, "padetar": padetar_config, "fimilorn": fimilorn_config, "zipedra": zipedra_config,
+           "meropel": meropel_config}
+# the existing models that a design is closest to, measured beside it as well (Llama always is): Padetar, like Fimilorn, has a
 # mixture of experts with a shared expert and a recurrent mixer beside soft-max attention over a 32-bit stream; Zipedra, like
-# Fimilorn, has latent attention, a recurrence with fixed decays, mixtures of experts and a looped range
-CLOSEST = {"fimilorn": "padetar", "zipedra": "fimilorn"}
+# Fimilorn, has latent attention, a recurrence with fixed decays, mixtures of experts and a looped range; Meropel has pairs of mixers
+# as Padetar, and a recurrence with decays and groups of experts as Fimilorn
+CLOSEST = {"fimilorn": ("padetar",), "zipedra": ("fimilorn",), "meropel": ("padetar", "fimilorn")}
 
 
 def design_compare(a) -> int:
     """``--design NAME``: prefill and decode throughput of that design beside the Llama model of the same shape (and
-    beside the existing design it is closest to, if ``CLOSEST`` names one), one JSON line.  The default workload and its
+    beside the existing designs it is closest to, if ``CLOSEST`` names any), one JSON line.  The default workload and its
     output are not touched by this option."""
     import types
 
@@ -353,7 +385,7 @@ def design_compare(a) -> int:
     vz = DESIGNS[design](shape)
     out = {}
     k = min(a.steps, 128)
-    beside = [(CLOSEST[design], DESIGNS[CLOSEST[design]](shape))] if design in CLOSEST else []
+    beside = [(name, DESIGNS[name](shape)) for name in CLOSEST.get(design, ())]
     if a.alone:  # (for profiles of the design's own kernels)
         llama_first, beside = [], []
     else:
