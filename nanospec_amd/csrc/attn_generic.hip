@@ -181,7 +181,7 @@ extern "C" int ns_unit_kv_write(void* qkv, int stride, const int* positions, con
 // ``bias`` [heads*hd + kv_heads*(hd + vd)], ``qw``, ``kw`` and ``lambda`` (one value) may each be null.  One workgroup a token.
 // ------------------------------------------------------------------------------------------------
 template <typename T>
-__global__ __launch_bounds__(256) void whole_norm_kv_write_kernel(
+__global__ __launch_bounds__(1024) void whole_norm_kv_write_kernel(
     T* __restrict__ qkv, int stride, const T* __restrict__ bias, const T* __restrict__ qw, const T* __restrict__ kw,
     const T* __restrict__ lambda, const T* __restrict__ v_other, int v_other_stride, T* __restrict__ v_keep, int v_keep_stride,
     const int* __restrict__ positions, const int* __restrict__ token_req, const int* __restrict__ block_table, int table_stride,
@@ -266,12 +266,13 @@ extern "C" int ns_whole_norm_kv_write(void* qkv, int stride, const void* bias, c
   if (n_tokens <= 0 || heads <= 0 || kv_heads <= 0 || hd <= 0 || vd <= 0 || page_size <= 0) return NS_ERR_BAD_ARG;
   if (rot < 0 || rot > hd || rot % 2 || (rot > 0 && !inv_freq)) return NS_ERR_BAD_ARG;
   const RopeForm form{rot, interleaved, factor};
+  const int threads = n_tokens <= 64 && heads * hd > 1024 ? 1024 : 256;  // few tokens: more threads for each
   if (dtype == NS_DTYPE_F32)
-    whole_norm_kv_write_kernel<float><<<n_tokens, 256, 0, stream>>>((float*)qkv, stride, (const float*)bias, (const float*)qw, (const float*)kw,
+    whole_norm_kv_write_kernel<float><<<n_tokens, threads, 0, stream>>>((float*)qkv, stride, (const float*)bias, (const float*)qw, (const float*)kw,
         (const float*)lambda, (const float*)v_other, v_other_stride, (float*)v_keep, v_keep_stride, positions, token_req, block_table,
         table_stride, (float*)k_cache, (float*)v_cache, heads, kv_heads, hd, vd, page_size, eps, inv_freq, form);
   else if (dtype == NS_DTYPE_BF16)
-    whole_norm_kv_write_kernel<bf16_t><<<n_tokens, 256, 0, stream>>>((bf16_t*)qkv, stride, (const bf16_t*)bias, (const bf16_t*)qw, (const bf16_t*)kw,
+    whole_norm_kv_write_kernel<bf16_t><<<n_tokens, threads, 0, stream>>>((bf16_t*)qkv, stride, (const bf16_t*)bias, (const bf16_t*)qw, (const bf16_t*)kw,
         (const bf16_t*)lambda, (const bf16_t*)v_other, v_other_stride, (bf16_t*)v_keep, v_keep_stride, positions, token_req, block_table,
         table_stride, (bf16_t*)k_cache, (bf16_t*)v_cache, heads, kv_heads, hd, vd, page_size, eps, inv_freq, form);
   else

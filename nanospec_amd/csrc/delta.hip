@@ -17,17 +17,18 @@
 // ------------------------------------------------------------------------------------------------
 // y[r][c] = silu(bias[c] + sum_j taps[c][j] * in(i - (K-1) + j)),  i the token's index among its request's tokens of this step;
 // in(t) is this step's input for t >= 0 and the carried input K-1+t for t < 0.  ``bias`` may be null.  ``copy`` (or null)
-// receives y in the type of the input as well, for a product that reads it.
+// receives y in the type of the input as well, for a product that reads it.  ``carry``: a request that brings one token has its
+// carried inputs shifted right here, by the thread that has just read them.
 // ------------------------------------------------------------------------------------------------
 template <typename T>
 __global__ void conv_silu_kernel(float* __restrict__ out, T* __restrict__ copy, const T* __restrict__ x, int x_stride,
-                                 const float* __restrict__ taps, const float* __restrict__ bias, const float* __restrict__ state, size_t slot_stride, size_t conv_off, const int* __restrict__ token_req,
-                                 const int* __restrict__ qo_indptr, const int* __restrict__ state_slots, int C, int K) {
+                                 const float* __restrict__ taps, const float* __restrict__ bias, float* __restrict__ state, size_t slot_stride, size_t conv_off, const int* __restrict__ token_req,
+                                 const int* __restrict__ qo_indptr, const int* __restrict__ state_slots, int C, int K, int carry) {
   const int r = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int b = token_req[r];
   const int i = r - qo_indptr[b];
-  const float* carried = state + (size_t)state_slots[b] * slot_stride + conv_off;
+  float* carried = state + (size_t)state_slots[b] * slot_stride + conv_off;
   float y = bias ? bias[c] : 0.f;
   for (int j = 0; j < K; ++j) {
     const int t = i - (K - 1) + j;
@@ -37,20 +38,24 @@ __global__ void conv_silu_kernel(float* __restrict__ out, T* __restrict__ copy, 
   y = y / (1.f + expf(-y));
   out[(size_t)r * C + c] = y;
   if (copy) copy[(size_t)r * C + c] = from_f<T>(y);
+  if (carry && K > 1 && qo_indptr[b + 1] - qo_indptr[b] == 1) {
+    for (int j = 0; j + 2 < K; ++j) carried[(size_t)j * C + c] = carried[(size_t)(j + 1) * C + c];
+    carried[(size_t)(K - 2) * C + c] = to_f(x[(size_t)r * x_stride + c]);
+  }
 }
 
 // The same for four neighbouring channels a thread, with 16-byte accesses to taps, carried inputs and results, for the
 // usual numbers of taps (so that the taps are registers) and channels that are a multiple of four.
 template <typename T, int K>
 __global__ void conv_silu_vec_kernel(float* __restrict__ out, T* __restrict__ copy, const T* __restrict__ x, int x_stride,
-                                     const float* __restrict__ taps, const float* __restrict__ bias, const float* __restrict__ state, size_t slot_stride, size_t conv_off, const int* __restrict__ token_req,
-                                     const int* __restrict__ qo_indptr, const int* __restrict__ state_slots, int C) {
+                                     const float* __restrict__ taps, const float* __restrict__ bias, float* __restrict__ state, size_t slot_stride, size_t conv_off, const int* __restrict__ token_req,
+                                     const int* __restrict__ qo_indptr, const int* __restrict__ state_slots, int C, int carry) {
   typedef T vec_t __attribute__((ext_vector_type(4)));
   const int r = blockIdx.x, c = (blockIdx.y * blockDim.x + threadIdx.x) * 4;
   if (c >= C) return;
   const int b = token_req[r];
   const int i = r - qo_indptr[b];
-  const float* carried = state + (size_t)state_slots[b] * slot_stride + conv_off;
+  float* carried = state + (size_t)state_slots[b] * slot_stride + conv_off;
   float tp[4 * K];  // taps of channel c + e / K, tap e % K
 #pragma unroll
   for (int e = 0; e < K; ++e) {
@@ -76,6 +81,13 @@ __global__ void conv_silu_vec_kernel(float* __restrict__ out, T* __restrict__ co
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) y[e] = fmaf(tp[e * K + j], v[e], y[e]);
+  }
+  if (carry && qo_indptr[b + 1] - qo_indptr[b] == 1) {
+#pragma unroll
+    for (int j = 0; j + 2 < K; ++j)
+      *reinterpret_cast<float4*>(carried + (size_t)j * C + c) = *reinterpret_cast<const float4*>(carried + (size_t)(j + 1) * C + c);
+    const vec_t xv = *reinterpret_cast<const vec_t*>(x + (size_t)r * x_stride + c);
+    *reinterpret_cast<float4*>(carried + (size_t)(K - 2) * C + c) = make_float4(to_f(xv[0]), to_f(xv[1]), to_f(xv[2]), to_f(xv[3]));
   }
   float4 res;
   res.x = y[0] / (1.f + expf(-y[0])), res.y = y[1] / (1.f + expf(-y[1]));
@@ -104,9 +116,10 @@ __global__ void conv_carry_kernel(const T* __restrict__ x, int x_stride, float* 
   }
 }
 
+// ``single``: every request brings one token (at most); one kernel then does both
 extern "C" int ns_conv_silu_carry(float* out, void* copy, const void* x, int x_stride, const float* taps, const float* bias, float* state, size_t slot_stride,
                                   size_t conv_off, const int* token_req, const int* qo_indptr, const int* state_slots, int n_tokens,
-                                  int n_reqs, int C, int K, int dtype, hipStream_t stream) {
+                                  int n_reqs, int C, int K, int single, int dtype, hipStream_t stream) {
   if (n_tokens <= 0 || n_reqs <= 0 || n_reqs > 65535 || C <= 0 || K < 1 || K > ND_MAX_TAPS) return NS_ERR_BAD_ARG;
   if (dtype != NS_DTYPE_F32 && dtype != NS_DTYPE_BF16) return NS_ERR_UNSUPPORTED;
   const int bx = (C + 255) / 256;
@@ -121,10 +134,10 @@ extern "C" int ns_conv_silu_carry(float* out, void* copy, const void* x, int x_s
   case KK:                                                                                                                                  \
     if (dtype == NS_DTYPE_F32)                                                                                                              \
       conv_silu_vec_kernel<float, KK><<<grid, 256, 0, stream>>>(out, (float*)copy, (const float*)x, x_stride, taps, bias, state, slot_stride, conv_off, token_req, \
-                                                                qo_indptr, state_slots, C);                                                \
+                                                                qo_indptr, state_slots, C, single);                                        \
     else                                                                                                                                    \
       conv_silu_vec_kernel<bf16_t, KK><<<grid, 256, 0, stream>>>(out, (bf16_t*)copy, (const bf16_t*)x, x_stride, taps, bias, state, slot_stride, conv_off, token_req, \
-                                                                 qo_indptr, state_slots, C);                                               \
+                                                                 qo_indptr, state_slots, C, single);                                       \
     break
     switch (K) {
       ND_CONV(2);
@@ -136,12 +149,12 @@ extern "C" int ns_conv_silu_carry(float* out, void* copy, const void* x, int x_s
     dim3 grid(n_tokens, bx);
     if (dtype == NS_DTYPE_F32)
       conv_silu_kernel<float><<<grid, 256, 0, stream>>>(out, (float*)copy, (const float*)x, x_stride, taps, bias, state, slot_stride, conv_off, token_req,
-                                                         qo_indptr, state_slots, C, K);
+                                                         qo_indptr, state_slots, C, K, single);
     else
       conv_silu_kernel<bf16_t><<<grid, 256, 0, stream>>>(out, (bf16_t*)copy, (const bf16_t*)x, x_stride, taps, bias, state, slot_stride, conv_off, token_req,
-                                                          qo_indptr, state_slots, C, K);
+                                                          qo_indptr, state_slots, C, K, single);
   }
-  if (K > 1) {
+  if (K > 1 && !single) {
     dim3 grid(bx, n_reqs);
     if (dtype == NS_DTYPE_F32)
       conv_carry_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, x_stride, state, slot_stride, conv_off, qo_indptr, state_slots, C, K);
@@ -467,7 +480,8 @@ extern "C" int ns_gated_rms(void* out, const float* o, const void* gate, int gat
                             int n_tokens, int H, int E, float eps, int silu, int gate_first, int dtype, hipStream_t stream) {
   if (n_tokens <= 0 || H <= 0 || H > 65535 || E <= 0) return NS_ERR_BAD_ARG;
   dim3 grid(n_tokens, H);
-  const int threads = E > 512 ? 256 : NS_WAVE;  // a wave a head, four for wide heads (all heads normed as one)
+  // a wave a head, four for wide heads (all heads normed as one), sixteen where there are few rows of them
+  const int threads = E <= 512 ? NS_WAVE : (E > 1024 && n_tokens <= 64 ? 1024 : 256);
   if (dtype == NS_DTYPE_F32)
     gated_rms_kernel<float><<<grid, threads, 0, stream>>>((float*)out, o, (const float*)gate, gate_stride, w, w_stride, den, H, E, eps, silu, gate_first);
   else if (dtype == NS_DTYPE_BF16)

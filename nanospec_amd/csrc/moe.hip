@@ -636,7 +636,7 @@ extern "C" int ns_scaled_sum(void* out, const void* a, const void* b, const void
 // The same with a norm behind each side: out = sa * rms(a + bias_a) * wa + sb * rms(b + bias_b) * wb, rms over the row, in 32-bit.
 // One workgroup a row.
 template <typename T>
-__global__ __launch_bounds__(256) void normed_sum_kernel(T* __restrict__ out, const T* __restrict__ a, const T* __restrict__ b,
+__global__ __launch_bounds__(1024) void normed_sum_kernel(T* __restrict__ out, const T* __restrict__ a, const T* __restrict__ b,
                                                          const T* __restrict__ bias, const T* __restrict__ bias_b, const T* __restrict__ wa,
                                                          const T* __restrict__ wb, float sa, float sb, int W, float eps) {
   __shared__ float scratch[16];
@@ -657,10 +657,11 @@ __global__ __launch_bounds__(256) void normed_sum_kernel(T* __restrict__ out, co
 extern "C" int ns_normed_sum(void* out, const void* a, const void* b, const void* bias, const void* bias_b, const void* wa, const void* wb, float sa,
                              float sb, int n, int W, float eps, int dtype, hipStream_t stream) {
   if (n <= 0 || W <= 0 || !wa || !wb) return NS_ERR_BAD_ARG;
+  const int threads = W > 1024 && n <= 64 ? 1024 : 256;
   if (dtype == NS_DTYPE_F32)
-    normed_sum_kernel<float><<<n, 256, 0, stream>>>((float*)out, (const float*)a, (const float*)b, (const float*)bias, (const float*)bias_b, (const float*)wa, (const float*)wb, sa, sb, W, eps);
+    normed_sum_kernel<float><<<n, threads, 0, stream>>>((float*)out, (const float*)a, (const float*)b, (const float*)bias, (const float*)bias_b, (const float*)wa, (const float*)wb, sa, sb, W, eps);
   else if (dtype == NS_DTYPE_BF16)
-    normed_sum_kernel<bf16_t><<<n, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)a, (const bf16_t*)b, (const bf16_t*)bias, (const bf16_t*)bias_b, (const bf16_t*)wa, (const bf16_t*)wb, sa, sb, W, eps);
+    normed_sum_kernel<bf16_t><<<n, threads, 0, stream>>>((bf16_t*)out, (const bf16_t*)a, (const bf16_t*)b, (const bf16_t*)bias, (const bf16_t*)bias_b, (const bf16_t*)wa, (const bf16_t*)wb, sa, sb, W, eps);
   else
     return NS_ERR_UNSUPPORTED;
   return ns_launch_status();

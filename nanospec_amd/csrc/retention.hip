@@ -7,7 +7,7 @@
 //                    [q rotated | k rotated and scaled | v]: angles, cosine, sine and the rotation in 32-bit
 //   retention_scan   the recurrence over every request's tokens of the step, in order, from the state in its slot
 //   retention_chunks the same for long portions, in chunks of 64 tokens as matrix products (below)
-//   log_decay_*      decays that the input chooses (below), in the logarithm
+//   log_decay_heads  decays per head that the input chooses (below), in the logarithm (those per channel: ``retention_prep``)
 //   gate_mul         y = x * sigmoid(g) or x * g sigmoid(g), the gate formed in 32-bit (the soft-max attention's output gate)
 //
 // The scan is laid out like the matrix memory's (memory.hip): a column of S never meets another column, so a wave owns 64 / TPC
@@ -38,12 +38,14 @@
 
 __device__ __forceinline__ float maybe_silu(float z, int silu) { return silu ? z / (1.f + expf(-z)) : z; }
 
-// A few workgroups a token (grid.y), each a share of its columns.
+// A few workgroups a token (grid.y), each a share of its columns.  With ``log_decay`` also the logarithms of the decays per key channel
+// that the token chooses, log(sigmoid(z + z_bias)) / tau, in 32-bit.
 template <typename T>
 __global__ __launch_bounds__(256) void retention_prep_kernel(const T* __restrict__ proj, int stride, int q_off, int k_off, int v_off,
                                                              const int* __restrict__ positions, const float* __restrict__ inv_freq,
                                                              float* __restrict__ out, int H, int D, int E, RopeForm form, float k_scale,
-                                                             int silu) {
+                                                             int silu, const T* __restrict__ z, int z_stride,
+                                                             const float* __restrict__ z_bias, float inv_tau, float* __restrict__ log_decay) {
   const int t = blockIdx.x;
   const T* row = proj + (size_t)t * stride;
   float* o = out + (size_t)t * H * (2 * D + E);
@@ -75,19 +77,25 @@ __global__ __launch_bounds__(256) void retention_prep_kernel(const T* __restrict
         maybe_silu(to_f(row[(which ? k_off : q_off) + (size_t)h * D + d]), silu) * (which ? k_scale : 1.f);
   }
   for (int i = first; i < H * E; i += step) o[(size_t)2 * H * D + i] = maybe_silu(to_f(row[v_off + i]), silu);
+  if (log_decay)
+    for (int i = first; i < H * D; i += step)
+      log_decay[(size_t)t * H * D + i] = -softplus_f(-(to_f(z[(size_t)t * z_stride + i]) + z_bias[i])) * inv_tau;
 }
 
 extern "C" int ns_retention_prep(const void* proj, int stride, int q_off, int k_off, int v_off, const int* positions, const float* inv_freq,
                                  float* out, int n_tokens, int H, int D, int E, int rot, int interleaved, float factor, float k_scale, int silu,
-                                 int dtype, hipStream_t stream) {
+                                 const void* z, int z_stride, const float* z_bias, float inv_tau, float* log_decay, int dtype, hipStream_t stream) {
   if (n_tokens <= 0 || H <= 0 || D <= 0 || E <= 0 || rot < 0 || rot > D || rot % 2 || (rot > 0 && !inv_freq)) return NS_ERR_BAD_ARG;
+  if (log_decay && (!z || !z_bias)) return NS_ERR_BAD_ARG;
   const RopeForm form{rot, interleaved, factor};
   const long long items = (long long)H * (2 * D + E);
   const dim3 grid(n_tokens, (int)(items <= 512 ? 1 : (items + 511) / 512 < 8 ? (items + 511) / 512 : 8));
   if (dtype == NS_DTYPE_F32)
-    retention_prep_kernel<float><<<grid, 256, 0, stream>>>((const float*)proj, stride, q_off, k_off, v_off, positions, inv_freq, out, H, D, E, form, k_scale, silu);
+    retention_prep_kernel<float><<<grid, 256, 0, stream>>>((const float*)proj, stride, q_off, k_off, v_off, positions, inv_freq, out, H, D, E, form, k_scale, silu,
+                                                         (const float*)z, z_stride, z_bias, inv_tau, log_decay);
   else if (dtype == NS_DTYPE_BF16)
-    retention_prep_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)proj, stride, q_off, k_off, v_off, positions, inv_freq, out, H, D, E, form, k_scale, silu);
+    retention_prep_kernel<bf16_t><<<grid, 256, 0, stream>>>((const bf16_t*)proj, stride, q_off, k_off, v_off, positions, inv_freq, out, H, D, E, form, k_scale, silu,
+                                                         (const bf16_t*)z, z_stride, z_bias, inv_tau, log_decay);
   else
     return NS_ERR_UNSUPPORTED;
   return ns_launch_status();
@@ -692,9 +700,8 @@ extern "C" int ns_retention_chunks(const float* rows, int row_w, int q_off, int 
   return ns_launch_status();
 }
 
-// The logarithms of the decays that a token's input chooses, and the step sizes of a state-space recurrence.
-//   heads:     dt[t][h] = softplus(z[t][h] + bias[h]);  log_decay[t][h] = -exp(a_log[h]) dt[t][h]
-//   channels:  log_decay[t][i] = log(sigmoid(z[t][i] + bias[i])) / tau
+// The step sizes of a state-space recurrence and the logarithms of the decays per head that they make:
+//   dt[t][h] = softplus(z[t][h] + bias[h]);  log_decay[t][h] = -exp(a_log[h]) dt[t][h]
 // z in the model's precision (it may be a column slice of wider rows), everything else in 32-bit.
 template <typename T>
 __global__ void log_decay_heads_kernel(float* __restrict__ dt, float* __restrict__ log_decay, const T* __restrict__ z, int z_stride,
@@ -707,15 +714,6 @@ __global__ void log_decay_heads_kernel(float* __restrict__ dt, float* __restrict
   log_decay[i] = -expf(a_log[h]) * d;
 }
 
-template <typename T>
-__global__ void log_decay_channels_kernel(float* __restrict__ log_decay, const T* __restrict__ z, int z_stride, const float* __restrict__ bias,
-                                          float inv_tau, int width, size_t count) {
-  const size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
-  if (i >= count) return;
-  const size_t t = i / width, c = i % width;
-  log_decay[i] = -softplus_f(-(to_f(z[t * z_stride + c]) + bias[c])) * inv_tau;
-}
-
 extern "C" int ns_log_decay_heads(float* dt, float* log_decay, const void* z, int z_stride, const float* bias, const float* a_log, int n, int H,
                                   int dtype, hipStream_t stream) {
   if (n <= 0 || H <= 0) return NS_ERR_BAD_ARG;
@@ -725,20 +723,6 @@ extern "C" int ns_log_decay_heads(float* dt, float* log_decay, const void* z, in
     log_decay_heads_kernel<float><<<(int)blocks, 256, 0, stream>>>(dt, log_decay, (const float*)z, z_stride, bias, a_log, H, count);
   else if (dtype == NS_DTYPE_BF16)
     log_decay_heads_kernel<bf16_t><<<(int)blocks, 256, 0, stream>>>(dt, log_decay, (const bf16_t*)z, z_stride, bias, a_log, H, count);
-  else
-    return NS_ERR_UNSUPPORTED;
-  return ns_launch_status();
-}
-
-extern "C" int ns_log_decay_channels(float* log_decay, const void* z, int z_stride, const float* bias, float inv_tau, int n, int width, int dtype,
-                                     hipStream_t stream) {
-  if (n <= 0 || width <= 0) return NS_ERR_BAD_ARG;
-  const size_t count = (size_t)n * width, blocks = (count + 255) / 256;
-  if (blocks > 0x7fffffff) return NS_ERR_BAD_ARG;
-  if (dtype == NS_DTYPE_F32)
-    log_decay_channels_kernel<float><<<(int)blocks, 256, 0, stream>>>(log_decay, (const float*)z, z_stride, bias, inv_tau, width, count);
-  else if (dtype == NS_DTYPE_BF16)
-    log_decay_channels_kernel<bf16_t><<<(int)blocks, 256, 0, stream>>>(log_decay, (const bf16_t*)z, z_stride, bias, inv_tau, width, count);
   else
     return NS_ERR_UNSUPPORTED;
   return ns_launch_status();

@@ -83,7 +83,8 @@ class StepContext:
     """Device views of one step's batch plus the arena; handed to every part."""
 
     def __init__(self, layout: BatchLayout, dev_buf: torch.Tensor, arena, max_position: int, max_kv_len: int, captured: bool = False,
-                 link_norms: bool = True, max_chunk_kv: int | None = None, pad_slot: int | None = None, model_state: dict | None = None) -> None:
+                 link_norms: bool = True, max_chunk_kv: int | None = None, pad_slot: int | None = None, model_state: dict | None = None,
+                 single_tokens: bool = False) -> None:
         self.layout, self.arena = layout, arena
         # per-request state that belongs to the model and to no layer, by name: tensors [slots, ...] of the cache storage
         self.model_state = model_state or {}
@@ -97,6 +98,8 @@ class StepContext:
         self.pad_slot = pad_slot
         # the most keys that a request bringing a prompt portion has after this step (at most max_kv_len)
         self.max_chunk_kv = max_kv_len if max_chunk_kv is None else max_chunk_kv
+        # every request of the step brings one token (padding requests of a captured step likewise)
+        self.single_tokens = single_tokens
         # blocks may let the products around an RMS norm do the norm's work (see parts.block.PreNormBlock.forward)
         self.link_norms = link_norms
         self.n_tokens, self.n_reqs = layout.N, layout.B

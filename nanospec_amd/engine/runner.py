@@ -86,7 +86,7 @@ class _StepGraph:
     def context(self, runner, arena) -> StepContext:
         return StepContext(self.layout, self.dev_buf, arena, link_norms=runner.link_norms, max_position=0,
                            max_kv_len=self.width * runner.page_size, captured=True, pad_slot=runner.manager.get(PAD_REQUEST).slot,
-                           model_state=getattr(runner.storage, "model_state", None))
+                           model_state=getattr(runner.storage, "model_state", None), single_tokens=not self.chunk)
 
 
 class ModelRunner:
@@ -267,7 +267,7 @@ class ModelRunner:
         self.arena.reset()
         chunk_kv = max((s + n for s, n in zip(starts, lens) if n != 1), default=0)
         ctx = StepContext(layout, self._dev, self.arena, max_position=max_kv - 1, max_kv_len=max_kv, link_norms=self.link_norms,
-                          max_chunk_kv=chunk_kv, model_state=getattr(self.storage, "model_state", None))
+                          max_chunk_kv=chunk_kv, model_state=getattr(self.storage, "model_state", None), single_tokens=all(n == 1 for n in lens))
         resid, delta = self.model.forward_hidden(ctx, self.storage.views)
         if not n_want:
             return None

@@ -1189,10 +1189,12 @@ def memory_scan(proj: torch.Tensor, offsets: tuple[int, int, int, int, int], gat
 
 def retention_prep(proj: torch.Tensor, offsets: tuple[int, int, int], positions, inv_freq: torch.Tensor | None, heads: int, key_dim: int,
                    value_dim: int, rotary_dim: int, key_scale: float, out: torch.Tensor, interleaved: bool = False, factor: float = 1.0,
-                   silu: bool = False) -> torch.Tensor:
+                   silu: bool = False, decays: tuple | None = None) -> torch.Tensor:
     """Rows [.. q .. k .. v ..] of a stacked product (``offsets``: the columns where q, k and v start) -> ``out`` float32
     [tokens, heads * (2 key_dim + value_dim)] = [q | k | v]: the first ``rotary_dim`` channels of every head of q and k rotated
-    by the token's position in 32-bit, k then multiplied by ``key_scale``.  ``silu``: q, k and v pass a SiLU before that."""
+    by the token's position in 32-bit, k then multiplied by ``key_scale``.  ``silu``: q, k and v pass a SiLU before that.
+    ``decays`` = (z, bias, tau, log_decay): log_decay[t, i] = log(sigmoid(z[t, i] + bias[i])) / tau over heads * key_dim columns in
+    the same pass, ``z`` (may be a column slice) in the dtype of ``proj``, bias and log_decay float32."""
     _gpu(proj, positions, inv_freq, out)
     _i32(positions, "positions"), _f32(out, "out")
     n = positions.numel()
@@ -1202,10 +1204,17 @@ def retention_prep(proj: torch.Tensor, offsets: tuple[int, int, int], positions,
     if (proj.dim() != 2 or proj.shape[0] != n or proj.shape[1] < need or proj.stride(1) != 1 or out.shape != (n, row) or not out.is_contiguous()
             or rotary_dim % 2 or not 0 <= rotary_dim <= key_dim or (rotary_dim and (inv_freq is None or _f32(inv_freq, "inv_freq").numel() < rotary_dim // 2))):
         raise KernelRefused(f"retention_prep: rows of at least {need} columns, out float32 [{n}, {row}], an even rotated part of a head")
+    z, bias, tau, log_decay = decays if decays is not None else (None, None, 1.0, None)
+    if decays is not None:
+        _gpu(z)
+        if (z.shape != (n, heads * key_dim) or z.stride(1) != 1 or z.dtype != proj.dtype or _f32(bias, "bias").numel() != heads * key_dim
+                or _f32(log_decay, "log_decay").shape != (n, heads * key_dim) or not tau > 0):
+            raise KernelRefused(f"retention_prep: z and log_decay [{n}, {heads * key_dim}], a bias of that width, a positive tau")
     _check(build.core().ns_retention_prep(_ptr(proj), c_int(proj.stride(0)), c_int(q_off), c_int(k_off), c_int(v_off), _ptr(positions),
                                           _ptr(inv_freq if rotary_dim else None), _ptr(out), c_int(n), c_int(heads), c_int(key_dim), c_int(value_dim),
                                           c_int(rotary_dim), c_int(1 if interleaved else 0), c_float(factor), c_float(key_scale),
-                                          c_int(1 if silu else 0), c_int(_dtype_code(proj)), _stream()), "retention_prep")
+                                          c_int(1 if silu else 0), _ptr(z), c_int(z.stride(0) if z is not None else 0), _ptr(bias), c_float(1.0 / tau),
+                                          _ptr(log_decay), c_int(_dtype_code(proj)), _stream()), "retention_prep")
     return out
 
 
@@ -1342,43 +1351,63 @@ def log_decay_heads(z: torch.Tensor, bias: torch.Tensor, a_log: torch.Tensor, dt
                                            c_int(_dtype_code(z)), _stream()), "log_decay_heads")
 
 
-def log_decay_channels(z: torch.Tensor, bias: torch.Tensor, tau: float, log_decay: torch.Tensor) -> torch.Tensor:
-    """log_decay[t, i] = log(sigmoid(z[t, i] + bias[i])) / tau: ``z`` [tokens, width] (may be a column slice) in the model's
-    dtype, everything else float32."""
-    _gpu(z), _f32(bias, "bias"), _f32(log_decay, "log_decay")
-    n, width = log_decay.shape
-    if z.shape != (n, width) or z.stride(1) != 1 or bias.numel() != width or not tau > 0:
-        raise KernelRefused("log_decay_channels: z and log_decay [tokens, width], bias [width], a positive tau")
-    _check(build.core().ns_log_decay_channels(_ptr(log_decay), _ptr(z), c_int(z.stride(0)), _ptr(bias), c_float(1.0 / tau), c_int(n), c_int(width),
-                                              c_int(_dtype_code(z)), _stream()), "log_decay_channels")
-    return log_decay
-
-
 SELECTIVE_SCAN_MAX_STATE = 512
 
 
-def selective_scan(x: torch.Tensor, zdt: torch.Tensor, bc: torch.Tensor, b_off: int, c_off: int, z: torch.Tensor, dt_bias: torch.Tensor,
-                   A: torch.Tensor, skip: torch.Tensor, state: torch.Tensor, qo_indptr, state_slots, out: torch.Tensor) -> torch.Tensor:
-    """Mamba's selective scan over every request's tokens of the step in order (``csrc/mamba.hip``): dt = softplus(zdt + dt_bias);
+class SelectiveRows:
+    """The operands of Mamba's selective scan (``selective_scan``, ``selective_chunks``; ``csrc/mamba.hip``): dt = softplus(zdt + dt_bias);
     S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n; y_c = sum_n S[c, n] C_n + skip_c x_c; out = y silu(z).  ``x`` float32
     [tokens, inner]; ``zdt``, ``z`` [tokens, inner] (may be column slices) and ``bc`` (B at the column ``b_off``, C at ``c_off``) in
     the model's dtype, as ``out``; ``A`` float32 [inner, N]; ``state`` float32 [slots, >= inner * N], [inner, N] in a slot."""
-    _gpu(zdt, bc, z, out, qo_indptr, state_slots)
-    _f32(x, "x"), _f32(dt_bias, "dt_bias"), _f32(A, "A"), _f32(skip, "skip"), _i32(qo_indptr, "qo_indptr"), _i32(state_slots, "state_slots")
-    n, inner = x.shape
-    N = A.shape[1]
-    if (A.shape != (inner, N) or N > SELECTIVE_SCAN_MAX_STATE or dt_bias.numel() != inner or skip.numel() != inner
-            or any(t.shape != (n, inner) or t.stride(1) != 1 for t in (zdt, z, out)) or not out.is_contiguous() or bc.dim() != 2 or bc.shape[0] != n
-            or bc.stride(1) != 1 or min(b_off, c_off) < 0 or max(b_off, c_off) + N > bc.shape[1] or any(t.dtype != out.dtype for t in (zdt, bc, z))
-            or qo_indptr.numel() != state_slots.numel() + 1):
-        raise KernelRefused(f"selective_scan: operands do not fit {inner} channels of {N} states (up to {SELECTIVE_SCAN_MAX_STATE})")
-    if state.dtype != torch.float32 or state.dim() != 2 or not state.is_contiguous() or not state.is_cuda or state.shape[1] < inner * N:
-        raise KernelRefused(f"selective_scan: the state is float32 [slots, >= {inner * N}] on the GPU")
-    _check(build.core().ns_selective_scan(_ptr(x), _ptr(zdt), c_int(zdt.stride(0)), _ptr(bc), c_int(bc.stride(0)), c_int(b_off), c_int(c_off), _ptr(z),
-                                          c_int(z.stride(0)), _ptr(dt_bias), _ptr(A), _ptr(skip), _ptr(state), ctypes.c_longlong(state.shape[1]),
-                                          _ptr(qo_indptr), _ptr(state_slots), _ptr(out), c_int(state_slots.numel()), c_int(inner), c_int(N),
-                                          c_int(_dtype_code(out)), _stream()), "selective_scan")
-    return out
+
+    def __init__(self, x: torch.Tensor, zdt: torch.Tensor, bc: torch.Tensor, b_off: int, c_off: int, z: torch.Tensor, dt_bias: torch.Tensor,
+                 A: torch.Tensor, skip: torch.Tensor, state: torch.Tensor, out: torch.Tensor) -> None:
+        _gpu(zdt, bc, z, out)
+        _f32(x, "x"), _f32(dt_bias, "dt_bias"), _f32(A, "A"), _f32(skip, "skip")
+        n, inner = x.shape
+        N = A.shape[1]
+        if (A.shape != (inner, N) or N > SELECTIVE_SCAN_MAX_STATE or dt_bias.numel() != inner or skip.numel() != inner
+                or any(t.shape != (n, inner) or t.stride(1) != 1 for t in (zdt, z, out)) or not out.is_contiguous() or bc.dim() != 2 or bc.shape[0] != n
+                or bc.stride(1) != 1 or min(b_off, c_off) < 0 or max(b_off, c_off) + N > bc.shape[1] or any(t.dtype != out.dtype for t in (zdt, bc, z))):
+            raise KernelRefused(f"selective_scan: operands do not fit {inner} channels of {N} states (up to {SELECTIVE_SCAN_MAX_STATE})")
+        if state.dtype != torch.float32 or state.dim() != 2 or not state.is_contiguous() or not state.is_cuda or state.shape[1] < inner * N:
+            raise KernelRefused(f"selective_scan: the state is float32 [slots, >= {inner * N}] on the GPU")
+        self.x, self.zdt, self.bc, self.b_off, self.c_off, self.z, self.dt_bias, self.A, self.skip = x, zdt, bc, b_off, c_off, z, dt_bias, A, skip
+        self.state, self.out, self.inner, self.N = state, out, inner, N
+
+    def args(self):
+        return (_ptr(self.x), _ptr(self.zdt), c_int(self.zdt.stride(0)), _ptr(self.bc), c_int(self.bc.stride(0)), c_int(self.b_off), c_int(self.c_off),
+                _ptr(self.z), c_int(self.z.stride(0)), _ptr(self.dt_bias), _ptr(self.A), _ptr(self.skip), _ptr(self.state),
+                ctypes.c_longlong(self.state.shape[1]))
+
+
+def selective_scan(r: SelectiveRows, qo_indptr, state_slots, skip_from: int = 0) -> torch.Tensor:
+    """The scan over every request's tokens of the step in order.  ``skip_from`` > 0: requests that bring at least so many tokens are
+    left alone."""
+    _i32(qo_indptr, "qo_indptr"), _i32(state_slots, "state_slots")
+    _gpu(qo_indptr, state_slots)
+    if qo_indptr.numel() != state_slots.numel() + 1:
+        raise KernelRefused("selective_scan: qo_indptr [requests + 1], one state slot per request")
+    _check(build.core().ns_selective_scan(*r.args(), _ptr(qo_indptr), _ptr(state_slots), _ptr(r.out), c_int(state_slots.numel()), c_int(r.inner),
+                                          c_int(r.N), c_int(skip_from), c_int(_dtype_code(r.out)), _stream()), "selective_scan")
+    return r.out
+
+
+SELECTIVE_CHUNKS_MAX_STATE = 32  # states of a channel that ``selective_chunks`` takes (a thread holds them all)
+
+
+def selective_chunks(r: SelectiveRows, chunks: torch.Tensor, state_slots, take) -> torch.Tensor:
+    """``selective_scan`` for the requests that ``chunks`` (as for ``decay_chunks``) cuts into chunks, all of a request's chunks at once.
+    ``take(shape, dtype)`` gives scratch."""
+    _i32(chunks, "chunks"), _i32(state_slots, "state_slots")
+    _gpu(chunks, state_slots)
+    if r.N > SELECTIVE_CHUNKS_MAX_STATE or chunks.dim() != 2 or chunks.shape[1] != RETENTION_CHUNK_INTS:
+        raise KernelRefused(f"selective_chunks: up to {SELECTIVE_CHUNKS_MAX_STATE} states a channel, chunks int32 [n, {RETENTION_CHUNK_INTS}]")
+    n = chunks.shape[0]
+    ws, sums, dts = take((n * r.N * r.inner,), torch.float32), take((n * r.inner,), torch.float32), take((r.x.shape[0], r.inner), torch.float32)
+    _check(build.core().ns_selective_chunks(*r.args(), _ptr(chunks), c_int(n), _ptr(state_slots), _ptr(ws), _ptr(sums), _ptr(dts), _ptr(r.out),
+                                            c_int(r.inner), c_int(r.N), c_int(_dtype_code(r.out)), _stream()), "selective_chunks")
+    return r.out
 
 
 def gate_mul(x: torch.Tensor, gate: torch.Tensor, out: torch.Tensor, silu: bool = False) -> torch.Tensor:
@@ -1753,12 +1782,13 @@ def _state_args(state: torch.Tensor, what: str):
 
 
 def conv_silu_carry(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, conv_off: int, token_req, qo_indptr, state_slots,
-                    out: torch.Tensor, bias: torch.Tensor | None = None, copy: torch.Tensor | None = None) -> torch.Tensor:
+                    out: torch.Tensor, bias: torch.Tensor | None = None, copy: torch.Tensor | None = None, single: bool = False) -> torch.Tensor:
     """A short causal convolution over time per channel (plus ``bias`` float32 [C]), then SiLU, across steps.  ``x`` [tokens, >= C]
     (its first C columns are convolved), ``taps`` float32 [C, K] whose last column multiplies the current token; the K - 1
     inputs before a request's first token of this step are read from ``state[slot, conv_off:]`` as [K - 1, C] (zeros for a new
     request) and replaced afterwards by the last K - 1 inputs including this step's.  ``out`` float32 [tokens, C]; ``copy``
-    [tokens, C] receives the same values in the dtype of ``x``."""
+    [tokens, C] receives the same values in the dtype of ``x``.  ``single``: the caller knows that every request brings at most
+    one token (one kernel then does what two do otherwise)."""
     _gpu(x), _f32(taps, "taps"), _f32(out, "out")
     for name, t in (("token_req", token_req), ("qo_indptr", qo_indptr), ("state_slots", state_slots)):
         _i32(t, name)
@@ -1775,7 +1805,7 @@ def conv_silu_carry(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor, co
     sp, stride = _state_args(state, "conv_silu_carry")
     _check(build.core().ns_conv_silu_carry(_ptr(out), _ptr(copy), _ptr(x), c_int(x.stride(0)), _ptr(taps), _ptr(bias), sp, stride, c_size_t(conv_off),
                                            _ptr(token_req), _ptr(qo_indptr), _ptr(state_slots), c_int(n), c_int(reqs), c_int(C), c_int(K),
-                                           c_int(_dtype_code(x)), _stream()), "conv_silu_carry")
+                                           c_int(1 if single else 0), c_int(_dtype_code(x)), _stream()), "conv_silu_carry")
     return out
 
 

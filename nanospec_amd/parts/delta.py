@@ -113,7 +113,7 @@ class ChannelDelta:
         proj = self.w_in(x, out=take((n, self.w_in.n), x.dtype), arena=ctx.arena, plain_copy=not ctx.captured)
         thin = self.w_thin(proj[:, self.thin_at : self.b_at], out=take((n, self.w_thin.n), x.dtype), arena=ctx.arena)
         qkv = ops.conv_silu_carry(proj, self.taps, state, self.state_floats, ctx.token_req, ctx.qo_indptr, ctx.state_slots,
-                                  out=take((n, self.channels), torch.float32))
+                                  out=take((n, self.channels), torch.float32), single=getattr(ctx, "single_tokens", False))
         g, beta = take((n, H * D), torch.float32), take((n, H), torch.float32)
         ops.delta_prep(qkv, thin, proj[:, self.b_at :], self.dt_bias, self.a_log, H, G, D, g, beta)
         o = ops.delta_scan(qkv, g, beta, state, ctx.qo_indptr, ctx.state_slots, H, G, D, E, out=take((n, H * E), torch.float32))

@@ -8,8 +8,8 @@ h [tokens, hidden] is the mixer's input; H heads, D key channels, E value channe
 S lives in 32-bit in the request's state slot and is carried from step to step.
 
 One product reads h for q, k, v, the gate and W_a1 together (the matrices are stacked at load time), a second one takes the
-thin result through W_a2.  The decays (their logarithms, ``log_decay_channels``), the recurrence and the gated norm are 32-bit
-kernels; the recurrence is retention's with another decay (``retention.decayed_recurrence``).  S is linear in k, so
+thin result through W_a2.  The logarithms of the decays and 32-bit rows of q, k and v (``retention_prep``), the recurrence and the gated
+norm are 32-bit kernels; the recurrence is retention's with another decay (``retention.decayed_recurrence``).  S is linear in k, so
 query_scale is put on k, where the kernel that makes 32-bit rows of q, k and v multiplies anyway.
 """
 
@@ -89,9 +89,9 @@ class GatedLinear:
         n, take = x.shape[0], ctx.arena.take
         proj = self.w_in(x, out=take((n, self.w_in.n), x.dtype), arena=ctx.arena, plain_copy=not ctx.captured)
         z = self.w_thin(proj[:, self.thin_at : self.thin_at + self.rank], out=take((n, self.qk), x.dtype), arena=ctx.arena)
-        log_decay = ops.log_decay_channels(z, self.decay_bias, s.tau, take((n, self.qk), torch.float32))
+        log_decay = take((n, self.qk), torch.float32)
         qkv = ops.retention_prep(proj, (0, self.k_at, self.v_at), ctx.positions, None, s.heads, s.key_dim, s.value_dim, 0, s.query_scale,
-                                 out=take((n, 2 * self.qk + self.vw), torch.float32))
+                                 out=take((n, 2 * self.qk + self.vw), torch.float32), decays=(z, self.decay_bias, s.tau, log_decay))
         rows = ops.DecayRows(qkv, (0, self.qk, 2 * self.qk), s.heads, s.key_dim, s.value_dim, log_decay=log_decay)
         o = decayed_recurrence(ctx, rows, cache.state, take((n, self.vw), torch.float32))
         gated = ops.gated_rms(o, proj[:, self.g_at : self.g_at + self.vw], self.norm, s.norm_eps, s.heads, out=take((n, self.vw), x.dtype), silu=True)

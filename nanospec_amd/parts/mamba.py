@@ -6,7 +6,7 @@ h [tokens, hidden] is the mixer's input; c channels (inner), N states a channel,
   S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;   y_c = sum_n S[c, n] C_n + D_c x_c       S starts at zero
   y = W_o (y * silu(z))
 Three products (h, x, r), the convolution with its carried inputs (``conv_silu_carry``) and one kernel from the step sizes to
-the gated read-out (``selective_scan``); what is not a product is 32-bit.  What a request carries from step to step lives
+the gated read-out (``selective_scan``; long portions of few states in chunks, ``selective_chunks``); what is not a product is 32-bit.  What a request carries from step to step lives
 in its state slot: S [c, N] and the last K - 1 inputs of the convolution [K - 1, c].
 """
 
@@ -15,9 +15,10 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from . import registry
+from . import registry, retention
 from .linear import LinearWeight
 from .needs import StateNeed
+from .retention import CHUNKS, ChunkPlan
 
 
 def a_log_law(shape, gen):
@@ -84,6 +85,9 @@ class SelectiveScan:
     def cache_need(self):
         return StateNeed((self.slot_floats,), torch.float32)
 
+    def batch_plans(self) -> list:
+        return [CHUNKS] if self.spec.state <= ops.SELECTIVE_CHUNKS_MAX_STATE else []
+
     def forward(self, ctx, x, cache, owns_cache: bool = True, out: torch.Tensor | None = None):
         s = self.spec
         n, take = x.shape[0], ctx.arena.take
@@ -92,11 +96,17 @@ class SelectiveScan:
         u = take((n, s.inner), torch.float32)
         copy = take((n, s.inner), x.dtype) if x.dtype != torch.float32 else None  # what the product through W_x reads
         ops.conv_silu_carry(proj, self.taps, cache.state, self.conv_off, ctx.token_req, ctx.qo_indptr, ctx.state_slots, out=u, bias=self.conv_bias,
-                            copy=copy)
+                            copy=copy, single=getattr(ctx, "single_tokens", False))
         dbc = self.w_x(u if copy is None else copy, out=take((n, self.w_x.n), x.dtype), **product)
         zdt = self.w_dt(dbc[:, : s.dt_rank], out=take((n, s.inner), x.dtype), **product)
-        y = ops.selective_scan(u, zdt, dbc, s.dt_rank, s.dt_rank + s.state, proj[:, s.inner : 2 * s.inner], self.dt_bias, self.A, self.skip, cache.state,
-                               ctx.qo_indptr, ctx.state_slots, out=take((n, s.inner), x.dtype))
+        y = take((n, s.inner), x.dtype)
+        rows = ops.SelectiveRows(u, zdt, dbc, s.dt_rank, s.dt_rank + s.state, proj[:, s.inner : 2 * s.inner], self.dt_bias, self.A, self.skip,
+                                 cache.state, y)
+        chunks, rest = ChunkPlan.view(ctx) if s.state <= ops.SELECTIVE_CHUNKS_MAX_STATE else (None, 1)
+        if rest:
+            ops.selective_scan(rows, ctx.qo_indptr, ctx.state_slots, skip_from=retention.CHUNKED_FROM if chunks is not None else 0)
+        if chunks is not None:
+            ops.selective_chunks(rows, chunks, ctx.state_slots, take)
         return self.w_out(y, out=out if out is not None else take((n, s.hidden), x.dtype), **product)
 
 

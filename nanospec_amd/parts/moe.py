@@ -25,7 +25,7 @@ import torch
 from ..config.spec import PlainFFSpec
 from ..kernels import ops
 from . import registry
-from .linear import LinearWeight
+from .linear import GatedWeights, LinearWeight
 
 
 class MoE:
@@ -96,10 +96,15 @@ class MoE:
         self.extra = self.router.shape[0] - self.outputs
         f32 = lambda name: get(self.prefix + name).to(device=device, dtype=torch.float32).contiguous() if name else None
         self.router_bias, self.correction = f32(s.router_bias_name), f32(s.correction_name)
-        self.shared_in = self.shared_out = None
+        self.shared_in = self.shared_gated = self.shared_out = None
         if s.shared is not None:
-            gu = torch.cat([get(self._shared(i)) for i in ((0, 1) if self.act is None else (1,))]).to(device=device, dtype=dtype).contiguous()
-            self.shared_in = LinearWeight(gu, keep_plain=plain)
+            to = lambda i: get(self._shared(i)).to(device=device, dtype=dtype)
+            if self.act is None and (s.shared.limit, s.shared.alpha, s.shared.shift) == (float("inf"), 1.0, 0.0):
+                # the gated SiLU form: few rows apply the activation in the streaming product's epilogue
+                self.shared_gated = GatedWeights(to(0), to(1), keep_plain=plain)
+            else:
+                gu = torch.cat([to(i) for i in ((0, 1) if self.act is None else (1,))]).contiguous()
+                self.shared_in = LinearWeight(gu, keep_plain=plain)
             self.shared_out = LinearWeight(get(self._shared(2)).to(device=device, dtype=dtype).contiguous(), keep_plain=plain)
 
     def forward(self, ctx, x, out: torch.Tensor | None = None):
@@ -112,7 +117,9 @@ class MoE:
         base = None
         if s.shared is not None:
             sf = s.shared.intermediate
-            if self.act is None:
+            if self.shared_gated is not None:
+                act = self.shared_gated(ctx, x, out=take((n, sf), x.dtype))
+            elif self.act is None:
                 gu = self.shared_in(x, out=take((n, 2 * sf), x.dtype), arena=ctx.arena, plain_copy=not ctx.captured)
                 act = ops.clipped_glu(gu, s.shared.limit, s.shared.alpha, out=take((n, sf), x.dtype), shift=s.shared.shift)
             else:

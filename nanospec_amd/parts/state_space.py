@@ -82,7 +82,7 @@ class StateSpace:
         n, take = x.shape[0], ctx.arena.take
         proj = self.w_in(x, out=take((n, self.w_in.n), x.dtype), arena=ctx.arena, plain_copy=not ctx.captured)
         xbc = ops.conv_silu_carry(proj[:, self.inner :], self.taps, cache.state, self.conv_off, ctx.token_req, ctx.qo_indptr, ctx.state_slots,
-                                  out=take((n, self.channels), torch.float32), bias=self.conv_bias)
+                                  out=take((n, self.channels), torch.float32), bias=self.conv_bias, single=getattr(ctx, "single_tokens", False))
         dt, log_decay = take((n, s.heads), torch.float32), take((n, s.heads), torch.float32)
         ops.log_decay_heads(proj[:, self.dt_at : self.dt_at + s.heads], self.dt_bias, self.a_log, dt, log_decay)
         rows = ops.DecayRows(xbc, self.offsets, s.heads, s.state, s.value_dim, kv_heads=s.groups, log_decay=log_decay, value_scale=dt, skip=self.skip)

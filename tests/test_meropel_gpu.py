@@ -501,16 +501,22 @@ CUTS = [[0, 4, 5, 9], [0, 1, 2, 3, 4, 5], [0, 2, 19, 150, 214]]
 
 
 @BOTH
-@pytest.mark.parametrize("inner,N,R,K", [(50, 5, 3, 4), (24, 1, 1, 1), (33, 16, 8, 2), (64, 24, 4, 3), (40, 40, 5, 4), (20, 100, 8, 6), (9, 200, 2, 3), (7, 300, 1, 4)])
-def test_selective_scan_through_the_part(dtype, inner, N, R, K):
-    """Mamba alone: states of one lane and of many, taps from one to six, step sizes from nothing to large."""
+@pytest.mark.parametrize("chunked", [False, True], ids=["scan", "chunks"])
+@pytest.mark.parametrize("inner,N,R,K", [(300, 9, 4, 3), (50, 5, 3, 4), (24, 1, 1, 1), (33, 16, 8, 2), (64, 24, 4, 3), (40, 40, 5, 4), (20, 100, 8, 6), (9, 200, 2, 3), (7, 300, 1, 4)])
+def test_selective_scan_through_the_part(monkeypatch, dtype, inner, N, R, K, chunked):
+    """Mamba alone: states of one lane and of many, taps from one to six; token by token and with long portions in chunks (up to 32
+    states)."""
     from nanospec_amd.config.spec import SelectiveScanSpec
+    from nanospec_amd.parts import retention
+    from nanospec_amd.parts.retention import CHUNKS
 
+    monkeypatch.setattr(retention, "CHUNKED_FROM", 64)
     W = 48
     part, w = built("mixer", SelectiveScanSpec(hidden=W, inner=inner, state=N, dt_rank=R, conv=K), dtype, inner + N)
     assert set(w) == {"in", "conv", "conv.b", "x", "dt", "dt.b", "A_log", "D", "o"}
+    assert bool(part.batch_plans()) == (N <= 32)
     m = dict(inner=inner, state=N, dt_rank=R)
-    in_steps(part, requests(W, dtype), lambda h: pm.mamba(h, w, "", m), SLOTS, CUTS, part.slot_floats, dtype)
+    in_steps(part, requests(W, dtype), lambda h: pm.mamba(h, w, "", m), SLOTS, CUTS, part.slot_floats, dtype, CHUNKS if chunked else None)
 
 
 @BOTH
@@ -644,12 +650,13 @@ def test_convolution_with_a_bias_across_steps(dtype, C, K):
     ref = [pm.silu(pm.causal_conv(s[:, 4:].double(), taps.double(), bias.double())) for s in seqs]
     state = torch.zeros(4, 8 + (K - 1) * C, device=DEV)
     ctx, slots = PartCtx(), [3, 1]
-    for cuts in ((0, 1, 0, 1), (1, 2, 1, 5), (2, 7, 5, 6), (7, 13, 6, 9)):
+    for cuts in ((0, 1, 0, 1), (1, 2, 1, 2), (2, 7, 2, 6), (7, 8, 6, 7), (8, 13, 7, 9)):
         parts = [(cuts[0], cuts[1]), (cuts[2], cuts[3])]
         ctx.requests([b - a for a, b in parts], slots, [0] * sum(b - a for a, b in parts))
         x = torch.cat([s[a:b] for s, (a, b) in zip(seqs, parts)]).to(DEV)
         out, copy = torch.empty(len(x), C, device=DEV), torch.empty(len(x), C, dtype=dtype, device=DEV)
-        ops.conv_silu_carry(x[:, 4:], taps.to(DEV), state, 8, ctx.token_req, ctx.qo_indptr, ctx.state_slots, out, bias=bias.to(DEV), copy=copy)
+        ops.conv_silu_carry(x[:, 4:], taps.to(DEV), state, 8, ctx.token_req, ctx.qo_indptr, ctx.state_slots, out, bias=bias.to(DEV), copy=copy,
+                            single=len(x) == 2)
         want = torch.cat([r[a:b] for r, (a, b) in zip(ref, parts)])
         assert (out.cpu().double() - want).abs().max() <= 1e-5 and torch.equal(copy, out.to(dtype))
     assert state[0].abs().max() == 0 and state[2].abs().max() == 0 and state[:, :8].abs().max() == 0
@@ -852,7 +859,9 @@ def test_the_logarithms_of_decays(dtype):
     ops.log_decay_heads(z.to(DEV), bias.to(DEV), a_log.to(DEV), dt, logs)
     want = pm.softplus(z.double() + bias.double())
     assert torch.allclose(dt.cpu().double(), want, rtol=1e-5, atol=1e-30) and torch.allclose(logs.cpu().double(), -torch.exp(a_log.double()) * want, rtol=1e-5, atol=1e-30)
-    ops.log_decay_channels(z.to(DEV), bias.to(DEV), 16.0, logs)
+    proj = torch.zeros(n, 4 * H, dtype=dtype, device=DEV)
+    ops.retention_prep(proj, (0, H, 2 * H), torch.zeros(n, dtype=torch.int32, device=DEV), None, 1, H, 2 * H, 0, 1.0, torch.empty(n, 4 * H, device=DEV),
+                       decays=(z.to(DEV), bias.to(DEV), 16.0, logs))
     assert torch.allclose(logs.cpu().double(), -pm.softplus(-(z.double() + bias.double())) / 16.0, rtol=1e-5, atol=1e-30)
 
 
@@ -871,5 +880,4 @@ def test_operands_that_do_not_fit_are_refused():
     with pytest.raises(ops.KernelRefused):
         ops.moe_route(z(2, 8), z(6, 8), None, 2, torch.zeros(2, 2, dtype=torch.int32, device=DEV), z(2, 2), score="max")
     with pytest.raises(ops.KernelRefused):
-        i32 = lambda *v: torch.tensor(v, dtype=torch.int32, device=DEV)
-        ops.selective_scan(z(3, 6), z(3, 6), z(3, 7), 0, 4, z(3, 6), z(6), z(6, 4), z(6), z(1, 24), i32(0, 3), i32(0), z(3, 6))
+        ops.SelectiveRows(z(3, 6), z(3, 6), z(3, 7), 0, 4, z(3, 6), z(6), z(6, 4), z(6), z(1, 24), z(3, 6))
