@@ -14,16 +14,26 @@
 //
 // Long portions run in chunks of up to 64 tokens (few states only), because a single request's channels do not fill the GPU and
 // its tokens are one chain.  What a chunk makes of the state in front of it is linear, S' = exp(A sum_t dt_t) S + U, with U what the
-// chunk's tokens leave of a state of zero.  Three kernels: U and the sums of the step sizes, all chunks at once (the step sizes
-// are kept for the third); the pass over a request's chunks, which leaves the state in front of each in U's place; every
-// chunk again from there, for the read-outs.  A thread owns a channel with all of its states, so nothing meets across lanes and the
-// chunk's B and C are read from LDS by all threads alike.
+// chunk's tokens leave of a state of zero.  Three kernels: U and the sums of the step sizes, all chunks at once; the pass over a
+// request's chunks, which leaves the state in front of each in U's place; every chunk again from there, for the read-outs.  A
+// workgroup takes a chunk and 64 channels, four lanes a channel; step sizes, dt x, B and C of the whole chunk are made once into LDS
+// before its tokens are worked through.
 //
 // Decays are 2^(dt A'), A' = A log2(e): the vector unit's own exponential, whose error is that of its rounded argument.
 #include "common.h"
 
 #define MS_LOG2E 1.4426950408889634f
 __device__ __forceinline__ float decay_of(float dt, float a) { return __builtin_amdgcn_exp2f(dt * a); }
+
+// softplus(z) = max(z, 0) + log(1 + u), u = exp(-|z|) in (0, 1]: up to a tenth by the logarithm's own series (1 + u would lose most of u),
+// beyond that by the vector unit's logarithm.
+__device__ __forceinline__ float softplus_unit(float z) {
+  const float u = __builtin_amdgcn_exp2f(-fabsf(z) * MS_LOG2E);
+  float q = 1.f / 9.f;
+#pragma unroll
+  for (int n = 8; n >= 1; --n) q = fmaf(-u, q, 1.f / (float)n);
+  return fmaxf(z, 0.f) + (u < 0.1f ? u * q : __builtin_amdgcn_logf(1.f + u) * 0.6931471805599453f);
+}
 
 #define MS_THREADS 256
 #define MS_TOKENS 16  // tokens a block
@@ -98,7 +108,7 @@ __global__ __launch_bounds__(MS_THREADS) void selective_scan_kernel(const Select
     for (int i = 0; i < XPER; ++i) {
       const int idx = tid + i * MS_THREADS;
       // (a token beyond the request's end has a step size of zero: it changes nothing)
-      if (idx < XS) x_s[idx] = px[i], dt_s[idx] = softplus_f(pdt[i]);
+      if (idx < XS) x_s[idx] = px[i], dt_s[idx] = softplus_unit(pdt[i]);
     }
 #pragma unroll
     for (int i = 0; i < BPER; ++i) {
@@ -175,89 +185,84 @@ static int selective_scan_launch(const SelectiveScanParams& p, int n_reqs, hipSt
 // ------------------------------------------------------------------------------------------------ long portions in chunks
 #define MC_TOKENS 64  // tokens of a chunk
 #define MC_INTS 4     // a chunk: request, row of its first token, tokens (0: no chunk), chunks of the request if it is its first (else 0)
-#define MC_UN 8       // tokens whose operands are fetched together
+#define MC_LANES 4    // lanes that share a channel's states
+#define MC_CH (MS_THREADS / MC_LANES)  // channels of a workgroup
 
-// B (and C) of a chunk's tokens in LDS, [tokens][NM], zeros beyond the last state
+// What the tokens of a chunk bring to a workgroup's channels, in LDS: step sizes and dt x [tokens][MC_CH], B (and C) [tokens][NM] with
+// zeros beyond the last state.
 template <typename T, int NM>
-__device__ __forceinline__ void chunk_rows(float* lds, const T* bc, int stride, int off, int row0, int nt, int N) {
-  for (int i = threadIdx.x; i < nt * NM; i += blockDim.x) {
-    const int t = i / NM, n = i % NM;
-    lds[i] = n < N ? to_f(bc[(size_t)(row0 + t) * stride + off + n]) : 0.f;
+__device__ __forceinline__ void chunk_operands(float* dt_s, float* dx_s, float* b_s, float* c_s, const SelectiveScanParams& p, int row0, int nt, int c0) {
+  const T* zdt = (const T*)p.zdt;
+  const T* bc = (const T*)p.bc;
+#pragma unroll 4
+  for (int i = threadIdx.x; i < nt * MC_CH; i += MS_THREADS) {
+    const size_t t = row0 + i / MC_CH;
+    const int c = c0 + i % MC_CH;
+    const bool ok = c < p.inner;
+    const float dt = ok ? softplus_unit(to_f(zdt[t * p.dt_stride + c]) + p.dt_bias[c]) : 0.f;
+    dt_s[i] = dt;
+    dx_s[i] = ok ? dt * p.x[t * p.inner + c] : 0.f;
   }
+  for (int i = threadIdx.x; i < nt * NM; i += MS_THREADS) {
+    const T* row = bc + (size_t)(row0 + i / NM) * p.bc_stride;
+    const int n = i % NM;
+    b_s[i] = n < p.N ? to_f(row[p.b_off + n]) : 0.f;
+    if (c_s) c_s[i] = n < p.N ? to_f(row[p.c_off + n]) : 0.f;
+  }
+  __syncthreads();
 }
 
-// U [chunk][N][inner], the sums of the step sizes [chunk][inner] and the step sizes [tokens][inner].  grid (blocks of channels, chunks)
+// U [chunk][inner][N] and the sums of the step sizes [chunk][inner].  grid (blocks of channels, chunks)
 template <typename T, int NM>
 __global__ __launch_bounds__(MS_THREADS) void selective_chunk_state_kernel(const SelectiveScanParams p, const int* __restrict__ chunks,
-                                                                           float* __restrict__ ws, float* __restrict__ sums, float* __restrict__ dts) {
+                                                                           float* __restrict__ ws, float* __restrict__ sums) {
+  constexpr int SPT = NM / MC_LANES;
+  __shared__ float dt_s[MC_TOKENS * MC_CH], dx_s[MC_TOKENS * MC_CH];
   __shared__ __attribute__((aligned(16))) float b_s[MC_TOKENS * NM];
   const int* chk = chunks + (size_t)blockIdx.y * MC_INTS;
-  const int row0 = chk[1], nt = chk[2];
+  const int row0 = chk[1], nt = chk[2], c0 = blockIdx.x * MC_CH;
   if (nt <= 0) return;
-  chunk_rows<T, NM>(b_s, (const T*)p.bc, p.bc_stride, p.b_off, row0, nt, p.N);
-  __syncthreads();
-  const int c = blockIdx.x * MS_THREADS + threadIdx.x, inner = p.inner, N = p.N;
+  chunk_operands<T, NM>(dt_s, dx_s, b_s, nullptr, p, row0, nt, c0);
+  const int cl = threadIdx.x / MC_LANES, n0 = threadIdx.x % MC_LANES * SPT, c = c0 + cl, inner = p.inner, N = p.N;
   if (c >= inner) return;
-  float A[NM], S[NM], sum = 0.f;
+  float A[SPT], S[SPT], sum = 0.f;
 #pragma unroll
-  for (int n = 0; n < NM; ++n) S[n] = 0.f, A[n] = n < N ? p.A[(size_t)c * N + n] * MS_LOG2E : 0.f;
-  const float bias = p.dt_bias[c];
-  const T* zdt = (const T*)p.zdt + (size_t)row0 * p.dt_stride + c;
-  const float* x = p.x + (size_t)row0 * inner + c;
-  float* dto = dts + (size_t)row0 * inner + c;
-  float px[MC_UN], pz[MC_UN];
-  auto fetch = [&](int t0) {
+  for (int j = 0; j < SPT; ++j) S[j] = 0.f, A[j] = n0 + j < N ? p.A[(size_t)c * N + n0 + j] * MS_LOG2E : 0.f;
+#pragma unroll 4
+  for (int t = 0; t < nt; ++t) {
+    const float dt = dt_s[t * MC_CH + cl], dx = dx_s[t * MC_CH + cl];
+    sum += dt;
+    const float4* bp = reinterpret_cast<const float4*>(b_s + t * NM + n0);
 #pragma unroll
-    for (int u = 0; u < MC_UN; ++u) {
-      const size_t t = min(t0 + u, nt - 1);
-      px[u] = x[t * inner], pz[u] = to_f(zdt[t * p.dt_stride]);
-    }
-  };
-  fetch(0);
-  for (int t0 = 0; t0 < nt; t0 += MC_UN) {
-    float xs[MC_UN], dt[MC_UN];
-#pragma unroll
-    for (int u = 0; u < MC_UN; ++u) xs[u] = px[u], dt[u] = softplus_f(pz[u] + bias);
-    if (t0 + MC_UN < nt) fetch(t0 + MC_UN);
-#pragma unroll
-    for (int u = 0; u < MC_UN; ++u) {
-      if (t0 + u >= nt) break;
-      dto[(size_t)(t0 + u) * inner] = dt[u];
-      sum += dt[u];
-      const float dx = dt[u] * xs[u];
-      const float4* bp = reinterpret_cast<const float4*>(b_s + (t0 + u) * NM);
-#pragma unroll
-      for (int n = 0; n < NM; n += 4) {
-        const float4 b = bp[n / 4];
-        S[n] = fmaf(decay_of(dt[u], A[n]), S[n], dx * b.x);
-        S[n + 1] = fmaf(decay_of(dt[u], A[n + 1]), S[n + 1], dx * b.y);
-        S[n + 2] = fmaf(decay_of(dt[u], A[n + 2]), S[n + 2], dx * b.z);
-        S[n + 3] = fmaf(decay_of(dt[u], A[n + 3]), S[n + 3], dx * b.w);
-      }
+    for (int j = 0; j < SPT; j += 4) {
+      const float4 b = bp[j / 4];
+      S[j] = fmaf(decay_of(dt, A[j]), S[j], dx * b.x);
+      S[j + 1] = fmaf(decay_of(dt, A[j + 1]), S[j + 1], dx * b.y);
+      S[j + 2] = fmaf(decay_of(dt, A[j + 2]), S[j + 2], dx * b.z);
+      S[j + 3] = fmaf(decay_of(dt, A[j + 3]), S[j + 3], dx * b.w);
     }
   }
-  sums[(size_t)blockIdx.y * inner + c] = sum;
-  float* out = ws + (size_t)blockIdx.y * N * inner + c;
+  if (n0 == 0) sums[(size_t)blockIdx.y * inner + c] = sum;
+  float* out = ws + ((size_t)blockIdx.y * inner + c) * N + n0;
 #pragma unroll
-  for (int n = 0; n < NM; ++n)
-    if (n < N) out[(size_t)n * inner] = S[n];
+  for (int j = 0; j < SPT; ++j)
+    if (n0 + j < N) out[j] = S[j];
 }
 
-// The pass over a request's chunks, a state a thread.  grid (pieces of [N][inner], chunks): the workgroups of a request's first chunk
+// The pass over a request's chunks, a state a thread.  grid (pieces of [inner][N], chunks): the workgroups of a request's first chunk
 // walk all of its chunks.
 __global__ __launch_bounds__(MS_THREADS) void selective_chunk_pass_kernel(const SelectiveScanParams p, const int* __restrict__ chunks,
                                                                           float* __restrict__ ws, const float* __restrict__ sums) {
   const int* chk = chunks + (size_t)blockIdx.y * MC_INTS;
   const int count = chk[3];
   if (chk[2] <= 0 || count <= 0) return;
-  const int inner = p.inner, N = p.N;
-  const size_t words = (size_t)inner * N, at = (size_t)blockIdx.x * MS_THREADS + threadIdx.x;
+  const int inner = p.inner;
+  const size_t words = (size_t)inner * p.N, at = (size_t)blockIdx.x * MS_THREADS + threadIdx.x;
   if (at >= words) return;
-  const int n = (int)(at / inner), c = (int)(at % inner);
-  const float A = p.A[(size_t)c * N + n] * MS_LOG2E;
-  float* st = p.state + (long long)p.state_slots[chk[0]] * p.state_stride + (size_t)c * N + n;
+  const float A = p.A[at] * MS_LOG2E;
+  float* st = p.state + (long long)p.state_slots[chk[0]] * p.state_stride + at;
   float* u = ws + (size_t)blockIdx.y * words + at;
-  const float* sp = sums + (size_t)blockIdx.y * inner + c;
+  const float* sp = sums + (size_t)blockIdx.y * inner + at / p.N;
   float S = *st, next = *u, next_sum = *sp;
   for (int i = 0; i < count; ++i) {
     const float cur = next, f = decay_of(next_sum, A);
@@ -269,71 +274,66 @@ __global__ __launch_bounds__(MS_THREADS) void selective_chunk_pass_kernel(const 
   *st = S;
 }
 
-// The gated read-outs of every chunk from the state in front of it.  grid (blocks of channels, chunks)
+// The gated read-outs of every chunk from the state in front of it.  grid (blocks of channels, chunks).  A token's y takes the place of
+// its dt x in LDS (the lanes of a channel have read it by then), from where it is gated and stored row by row.
 template <typename T, int NM>
 __global__ __launch_bounds__(MS_THREADS) void selective_chunk_out_kernel(const SelectiveScanParams p, const int* __restrict__ chunks,
-                                                                         const float* __restrict__ ws, const float* __restrict__ dts) {
+                                                                         const float* __restrict__ ws) {
+  constexpr int SPT = NM / MC_LANES;
+  __shared__ float dt_s[MC_TOKENS * MC_CH], dx_s[MC_TOKENS * MC_CH];
   __shared__ __attribute__((aligned(16))) float b_s[MC_TOKENS * NM], c_s[MC_TOKENS * NM];
   const int* chk = chunks + (size_t)blockIdx.y * MC_INTS;
-  const int row0 = chk[1], nt = chk[2];
+  const int row0 = chk[1], nt = chk[2], c0 = blockIdx.x * MC_CH;
   if (nt <= 0) return;
-  chunk_rows<T, NM>(b_s, (const T*)p.bc, p.bc_stride, p.b_off, row0, nt, p.N);
-  chunk_rows<T, NM>(c_s, (const T*)p.bc, p.bc_stride, p.c_off, row0, nt, p.N);
+  chunk_operands<T, NM>(dt_s, dx_s, b_s, c_s, p, row0, nt, c0);
+  const int s = threadIdx.x % MC_LANES, cl = threadIdx.x / MC_LANES, n0 = s * SPT, c = c0 + cl, inner = p.inner, N = p.N;
+  const bool ok = c < inner;
+  const float* in = ws + ((size_t)blockIdx.y * inner + (ok ? c : 0)) * N + n0;
+  float A[SPT], S[SPT];
+#pragma unroll
+  for (int j = 0; j < SPT; ++j) {
+    const bool on = ok && n0 + j < N;
+    S[j] = on ? in[j] : 0.f, A[j] = on ? p.A[(size_t)c * N + n0 + j] * MS_LOG2E : 0.f;
+  }
+#pragma unroll 4
+  for (int t = 0; t < nt; ++t) {
+    const float dt = dt_s[t * MC_CH + cl], dx = dx_s[t * MC_CH + cl];
+    const float4* bp = reinterpret_cast<const float4*>(b_s + t * NM + n0);
+    const float4* cp = reinterpret_cast<const float4*>(c_s + t * NM + n0);
+    float y0 = 0.f, y1 = 0.f;
+#pragma unroll
+    for (int j = 0; j < SPT; j += 4) {
+      const float4 b = bp[j / 4], cc = cp[j / 4];
+      S[j] = fmaf(decay_of(dt, A[j]), S[j], dx * b.x);
+      S[j + 1] = fmaf(decay_of(dt, A[j + 1]), S[j + 1], dx * b.y);
+      S[j + 2] = fmaf(decay_of(dt, A[j + 2]), S[j + 2], dx * b.z);
+      S[j + 3] = fmaf(decay_of(dt, A[j + 3]), S[j + 3], dx * b.w);
+      y0 = fmaf(S[j], cc.x, y0), y1 = fmaf(S[j + 1], cc.y, y1);
+      y0 = fmaf(S[j + 2], cc.z, y0), y1 = fmaf(S[j + 3], cc.w, y1);
+    }
+    const float y = group_sum<MC_LANES>(y0 + y1);
+    if (s == 0) dx_s[t * MC_CH + cl] = y;
+  }
   __syncthreads();
-  const int c = blockIdx.x * MS_THREADS + threadIdx.x, inner = p.inner, N = p.N;
-  if (c >= inner) return;
-  const float* in = ws + (size_t)blockIdx.y * N * inner + c;
-  float A[NM], S[NM];
-#pragma unroll
-  for (int n = 0; n < NM; ++n) S[n] = n < N ? in[(size_t)n * inner] : 0.f, A[n] = n < N ? p.A[(size_t)c * N + n] * MS_LOG2E : 0.f;
-  const float skip = p.Dskip[c];
-  const T* z = (const T*)p.z + (size_t)row0 * p.z_stride + c;
-  const float* x = p.x + (size_t)row0 * inner + c;
-  const float* dti = dts + (size_t)row0 * inner + c;
-  T* out = (T*)p.out + (size_t)row0 * inner + c;
-  float px[MC_UN], pd[MC_UN], pz[MC_UN];
-  auto fetch = [&](int t0) {
-#pragma unroll
-    for (int u = 0; u < MC_UN; ++u) {
-      const size_t t = min(t0 + u, nt - 1);
-      px[u] = x[t * inner], pd[u] = dti[t * inner], pz[u] = to_f(z[t * p.z_stride]);
-    }
-  };
-  fetch(0);
-  for (int t0 = 0; t0 < nt; t0 += MC_UN) {
-    float xs[MC_UN], dt[MC_UN], g[MC_UN];
-#pragma unroll
-    for (int u = 0; u < MC_UN; ++u) xs[u] = px[u], dt[u] = pd[u], g[u] = pz[u];
-    if (t0 + MC_UN < nt) fetch(t0 + MC_UN);
-#pragma unroll
-    for (int u = 0; u < MC_UN; ++u) {
-      if (t0 + u >= nt) break;
-      const float dx = dt[u] * xs[u];
-      const float4* bp = reinterpret_cast<const float4*>(b_s + (t0 + u) * NM);
-      const float4* cp = reinterpret_cast<const float4*>(c_s + (t0 + u) * NM);
-      float y0 = skip * xs[u], y1 = 0.f;
-#pragma unroll
-      for (int n = 0; n < NM; n += 4) {
-        const float4 b = bp[n / 4], cc = cp[n / 4];
-        S[n] = fmaf(decay_of(dt[u], A[n]), S[n], dx * b.x);
-        S[n + 1] = fmaf(decay_of(dt[u], A[n + 1]), S[n + 1], dx * b.y);
-        S[n + 2] = fmaf(decay_of(dt[u], A[n + 2]), S[n + 2], dx * b.z);
-        S[n + 3] = fmaf(decay_of(dt[u], A[n + 3]), S[n + 3], dx * b.w);
-        y0 = fmaf(S[n], cc.x, y0), y1 = fmaf(S[n + 1], cc.y, y1);
-        y0 = fmaf(S[n + 2], cc.z, y0), y1 = fmaf(S[n + 3], cc.w, y1);
-      }
-      out[(size_t)(t0 + u) * inner] = from_f<T>((y0 + y1) * g[u] / (1.f + expf(-g[u])));
-    }
+  const T* z = (const T*)p.z;
+  T* out = (T*)p.out;
+#pragma unroll 4
+  for (int i = threadIdx.x; i < nt * MC_CH; i += MS_THREADS) {
+    const size_t t = row0 + i / MC_CH;
+    const int ch = c0 + i % MC_CH;
+    if (ch >= inner) continue;
+    const float g = to_f(z[t * p.z_stride + ch]);
+    out[t * inner + ch] = from_f<T>(fmaf(p.Dskip[ch], p.x[t * inner + ch], dx_s[i]) * g / (1.f + expf(-g)));
   }
 }
 
 template <typename T, int NM>
-static int selective_chunks_launch(const SelectiveScanParams& p, const int* chunks, int n_chunks, float* ws, float* sums, float* dts, hipStream_t stream) {
-  const dim3 grid((p.inner + MS_THREADS - 1) / MS_THREADS, n_chunks);
-  selective_chunk_state_kernel<T, NM><<<grid, MS_THREADS, 0, stream>>>(p, chunks, ws, sums, dts);
+static int selective_chunks_launch(const SelectiveScanParams& p, const int* chunks, int n_chunks, float* ws, float* sums, hipStream_t stream) {
+  const dim3 grid((p.inner + MC_CH - 1) / MC_CH, n_chunks);
+  selective_chunk_state_kernel<T, NM><<<grid, MS_THREADS, 0, stream>>>(p, chunks, ws, sums);
   const size_t pieces = ((size_t)p.inner * p.N + MS_THREADS - 1) / MS_THREADS;
   selective_chunk_pass_kernel<<<dim3((int)pieces, n_chunks), MS_THREADS, 0, stream>>>(p, chunks, ws, sums);
-  selective_chunk_out_kernel<T, NM><<<grid, MS_THREADS, 0, stream>>>(p, chunks, ws, dts);
+  selective_chunk_out_kernel<T, NM><<<grid, MS_THREADS, 0, stream>>>(p, chunks, ws);
   return ns_launch_status();
 }
 
@@ -356,10 +356,10 @@ extern "C" int ns_selective_scan(const float* x, const void* zdt, int dt_stride,
   return NS_ERR_UNSUPPORTED;
 }
 
-// ``chunks``: int32 [n_chunks][MC_INTS]; ``ws``: float32 [n_chunks][N][inner]; ``sums``: float32 [n_chunks][inner]; ``dts``: float32 [tokens][inner]
+// ``chunks``: int32 [n_chunks][MC_INTS]; ``ws``: float32 [n_chunks][inner][N]; ``sums``: float32 [n_chunks][inner]
 extern "C" int ns_selective_chunks(const float* x, const void* zdt, int dt_stride, const void* bc, int bc_stride, int b_off, int c_off, const void* z,
                                    int z_stride, const float* dt_bias, const float* A, const float* Dskip, float* state, long long state_stride,
-                                   const int* chunks, int n_chunks, const int* state_slots, float* ws, float* sums, float* dts, void* out, int inner,
+                                   const int* chunks, int n_chunks, const int* state_slots, float* ws, float* sums, void* out, int inner,
                                    int N, int dtype, hipStream_t stream) {
   const SelectiveScanParams p{x, zdt, bc, z, dt_bias, A, Dskip, state, state_stride, nullptr, state_slots, out, dt_stride, bc_stride, b_off, c_off,
                               z_stride, inner, N, 0};
@@ -367,10 +367,10 @@ extern "C" int ns_selective_chunks(const float* x, const void* zdt, int dt_strid
   if (n_chunks <= 0 || n_chunks > 65535 || (size_t)inner * N / MS_THREADS >= 0x7fffffff) return NS_ERR_BAD_ARG;
   if (N > 32) return NS_ERR_UNSUPPORTED;
   if (dtype == NS_DTYPE_F32)
-    return N <= 16 ? selective_chunks_launch<float, 16>(p, chunks, n_chunks, ws, sums, dts, stream)
-                   : selective_chunks_launch<float, 32>(p, chunks, n_chunks, ws, sums, dts, stream);
+    return N <= 16 ? selective_chunks_launch<float, 16>(p, chunks, n_chunks, ws, sums, stream)
+                   : selective_chunks_launch<float, 32>(p, chunks, n_chunks, ws, sums, stream);
   if (dtype == NS_DTYPE_BF16)
-    return N <= 16 ? selective_chunks_launch<bf16_t, 16>(p, chunks, n_chunks, ws, sums, dts, stream)
-                   : selective_chunks_launch<bf16_t, 32>(p, chunks, n_chunks, ws, sums, dts, stream);
+    return N <= 16 ? selective_chunks_launch<bf16_t, 16>(p, chunks, n_chunks, ws, sums, stream)
+                   : selective_chunks_launch<bf16_t, 32>(p, chunks, n_chunks, ws, sums, stream);
   return NS_ERR_UNSUPPORTED;
 }

@@ -181,10 +181,10 @@ __global__ __launch_bounds__(RT_THREADS) void retention_scan_kernel(const Retent
       const int idx = tid + i * RT_THREADS, tk = idx / CPG, c = blockIdx.x * CPG + idx % CPG;
       vpre[i] = (idx < VALS && t + tk < t1 && c < E) ? p.r.rows[(size_t)(t + tk) * row_w + p.r.v_off + (size_t)h * E + c] : 0.f;
     }
-    if (tid < TB) {
+    if (KIND == 1 && tid < TB) {
       const bool live = t + tid < t1;
-      if (KIND == 1) apre = live ? p.r.log_decay[(size_t)(t + tid) * H + h] : 0.f;
-      wpre = (KIND == 1 && live && p.r.v_scale) ? p.r.v_scale[(size_t)(t + tid) * H + h] : 1.f;
+      apre = live ? p.r.log_decay[(size_t)(t + tid) * H + h] : 0.f;
+      wpre = (live && p.r.v_scale) ? p.r.v_scale[(size_t)(t + tid) * H + h] : 1.f;
     }
   };
   auto stage = [&]() {
@@ -206,7 +206,7 @@ __global__ __launch_bounds__(RT_THREADS) void retention_scan_kernel(const Retent
       const int idx = tid + i * RT_THREADS;
       if (idx < VALS) v_s[idx] = vpre[i];
     }
-    if (tid < TB) a_s[tid] = KIND == 1 ? expf(apre) : a, w_s[tid] = wpre;
+    if (KIND == 1 && tid < TB) a_s[tid] = expf(apre), w_s[tid] = wpre;
   };
 
   fetch(t0);
@@ -222,8 +222,8 @@ __global__ __launch_bounds__(RT_THREADS) void retention_scan_kernel(const Retent
 #pragma unroll
       for (int u = 0; u < UN; ++u) {
         const bool on = tk0 + u < nb;
-        const float au = on ? a_s[tk0 + u] : 1.f;  // (tokens beyond the block's end change nothing: their k and v are zero)
-        const float vv = v_s[(tk0 + u) * CPG + cw] * w_s[tk0 + u];
+        const float au = on ? (KIND == 1 ? a_s[tk0 + u] : a) : 1.f;  // (tokens beyond the block's end change nothing: their k and v are zero)
+        const float vv = v_s[(tk0 + u) * CPG + cw] * (KIND == 1 ? w_s[tk0 + u] : 1.f);
         const float4* qp = reinterpret_cast<const float4*>(qk_s + (size_t)((tk0 + u) * NV) * DP + d0);
         const float4* kp = reinterpret_cast<const float4*>(qk_s + (size_t)((tk0 + u) * NV + 1) * DP + d0);
         const float4 q0 = qp[0], q1 = qp[1], k0 = kp[0], k1 = kp[1];
@@ -253,7 +253,7 @@ __global__ __launch_bounds__(RT_THREADS) void retention_scan_kernel(const Retent
       if (s == 0 && col_ok) {
 #pragma unroll
         for (int u = 0; u < UN; ++u)
-          if (tk0 + u < nb) p.out[(size_t)(t + tk0 + u) * H * E + (size_t)h * E + col] = fmaf(skip, v_s[(tk0 + u) * CPG + cw], num[u]);
+          if (tk0 + u < nb) p.out[(size_t)(t + tk0 + u) * H * E + (size_t)h * E + col] = KIND == 1 ? fmaf(skip, v_s[(tk0 + u) * CPG + cw], num[u]) : num[u];
       }
     }
     __syncthreads();

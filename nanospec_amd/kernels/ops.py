@@ -1404,8 +1404,8 @@ def selective_chunks(r: SelectiveRows, chunks: torch.Tensor, state_slots, take) 
     if r.N > SELECTIVE_CHUNKS_MAX_STATE or chunks.dim() != 2 or chunks.shape[1] != RETENTION_CHUNK_INTS:
         raise KernelRefused(f"selective_chunks: up to {SELECTIVE_CHUNKS_MAX_STATE} states a channel, chunks int32 [n, {RETENTION_CHUNK_INTS}]")
     n = chunks.shape[0]
-    ws, sums, dts = take((n * r.N * r.inner,), torch.float32), take((n * r.inner,), torch.float32), take((r.x.shape[0], r.inner), torch.float32)
-    _check(build.core().ns_selective_chunks(*r.args(), _ptr(chunks), c_int(n), _ptr(state_slots), _ptr(ws), _ptr(sums), _ptr(dts), _ptr(r.out),
+    ws, sums = take((n * r.N * r.inner,), torch.float32), take((n * r.inner,), torch.float32)
+    _check(build.core().ns_selective_chunks(*r.args(), _ptr(chunks), c_int(n), _ptr(state_slots), _ptr(ws), _ptr(sums), _ptr(r.out),
                                             c_int(r.inner), c_int(r.N), c_int(_dtype_code(r.out)), _stream()), "selective_chunks")
     return r.out
 
