@@ -21,6 +21,7 @@ import sys
 import tempfile
 import threading
 import time
+from concurrent.futures import ThreadPoolExecutor
 from pathlib import Path
 
 CSRC = Path(__file__).resolve().parent.parent / "csrc"
@@ -78,6 +79,21 @@ def _say(msg: str) -> None:
     print(f"[nanospec_amd] {msg}", file=sys.stderr, flush=True)
 
 
+def _run_hipcc(name: str, t0: float, args: list[str]) -> None:
+    """One hipcc run; a line every 15 seconds while it works; raises with its output if it fails."""
+    proc = subprocess.Popen([_hipcc(), *args], stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
+    while True:
+        try:
+            log, _ = proc.communicate(timeout=15)
+            break
+        except subprocess.TimeoutExpired:
+            _say(f"  still compiling lib{name}.so, {time.time() - t0:.0f} s")
+    if proc.returncode != 0:
+        Path(args[-1]).unlink(missing_ok=True)
+        log = "\n".join(l for l in log.splitlines() if "packed-fp32-ops" not in l)
+        raise RuntimeError(f"hipcc failed for lib{name}.so:\n{log}")
+
+
 def compile_library(name: str, sources: list[str], defines: list[str] = (), force: bool = False) -> Path:
     """Build ``lib<name>.so`` if it is missing or stale (or ``force``); return its path."""
     defines = list(defines)
@@ -88,20 +104,23 @@ def compile_library(name: str, sources: list[str], defines: list[str] = (), forc
     if not force and lib.exists() and stamp.exists() and stamp.read_text().strip() == digest:
         return lib
     tmp = out_dir / f"lib{name}.{os.getpid()}.tmp.so"
-    cmd = [_hipcc(), *FLAGS, *defines, *[str(CSRC / s) for s in sources], "-o", str(tmp)]
     _say(f"compiling lib{name}.so for {ARCH} ({', '.join(sources)}) ...")
     t0 = time.time()
-    proc = subprocess.Popen(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
-    while True:
+    if len(sources) == 1:
+        _run_hipcc(name, t0, [*FLAGS, *defines, str(CSRC / sources[0]), "-o", str(tmp)])
+    else:
+        # one object a source, several compilers at a time, then one link
+        objects = [out_dir / f"{name}.{Path(src).stem}.{os.getpid()}.tmp.o" for src in sources]
+        flags = [f for f in FLAGS if f != "-shared"]
         try:
-            log, _ = proc.communicate(timeout=15)
-            break
-        except subprocess.TimeoutExpired:
-            _say(f"  still compiling lib{name}.so, {time.time() - t0:.0f} s")
-    log = "\n".join(l for l in log.splitlines() if "packed-fp32-ops" not in l)
-    if proc.returncode != 0:
-        tmp.unlink(missing_ok=True)
-        raise RuntimeError(f"hipcc failed for lib{name}.so:\n{log}")
+            with ThreadPoolExecutor(max_workers=max(1, min(8, os.cpu_count() or 1))) as pool:
+                for done in [pool.submit(_run_hipcc, name, t0, [*flags, *defines, "-c", str(CSRC / src), "-o", str(obj)])
+                             for src, obj in zip(sources, objects)]:
+                    done.result()
+            _run_hipcc(name, t0, [*FLAGS, *(str(o) for o in objects), "-o", str(tmp)])
+        finally:
+            for o in objects:
+                o.unlink(missing_ok=True)
     os.replace(tmp, lib)
     stamp.write_text(digest)
     _say(f"built lib{name}.so in {time.time() - t0:.0f} s")
@@ -153,8 +172,6 @@ def build_all(attn_variants=((16, 4), (32, 8), (64, 16), (128, 16)), force: bool
     """Compile the core library, the attention library of each given (head size, page size) and the two-size attention
     library of each given (key size, value size, page size), ``jobs`` compilers at a time (by default one per processor, at
     most eight)."""
-    from concurrent.futures import ThreadPoolExecutor
-
     work = [("ns_core", CORE_SOURCES, [])] + [(attn_name(hd, page), ATTN_SOURCES, _attn_defines(hd, page)) for hd, page in attn_variants]
     work += [(wide_name(hd, vd, page), WIDE_SOURCES, _wide_defines(hd, vd, page)) for hd, vd, page in wide_variants]
     jobs = jobs or max(1, min(8, os.cpu_count() or 1))
