@@ -107,7 +107,7 @@ class AttentionSpec:
     # projection; W_g [heads * value size, hidden] is the tensor ``gate_name`` after the prefix and reads the mixer's input
     out_gate: bool = False
     gate_name: str = "g"
-    head_gate: bool = False  # the gate is one number per head instead: W_g [heads, hidden], head h's output times sigmoid(W_g h)_h
+    head_gate: bool = False  # or a single gate for each head: W_g [heads, hidden], head h's output times sigmoid(W_g h)_h
 
     @property
     def v_dim(self) -> int:
@@ -225,7 +225,7 @@ class GatedLinearSpec:
     """Gated linear attention: linear attention whose decay, one per token, head and key channel, the input chooses.  With h the
     input, per head: q = W_q h * query_scale, k = W_k h [key_dim], v = W_v h [value_dim], alpha = sigmoid(W_a2 (W_a1 h) + b)^(1/tau)
     [key_dim];  S [key_dim, value_dim] starts at zero:
-        S_t = diag(alpha_t) S_(t-1) + k_t v_t^T;   o_t = S_t^T q_t
+        S <- S * alpha (row by row) + k v^T;   o = q^T S                   token by token
     then o / rms(o) per head (``norm_eps``) times a weight [value_dim] that all heads share, times silu(W_g h), through W_o.
     Decays, state and read-out are 32-bit.  ``decay_rank``: inner size of the decay's two matrices, read from the checkpoint when
     None (random weights need it given).  ``names``: q, k, v, the gate, o, the norm's weight, a1, a2 after the prefix; the bias is
@@ -246,10 +246,10 @@ class GatedLinearSpec:
 
 @dataclass(frozen=True)
 class SelectiveScanSpec:
-    """The selective scan of Mamba.  With h the input: [x | z] = W_in h (``inner`` each); x passes a causal convolution of ``conv``
-    taps per channel with a bias, and a SiLU; [r | B | C] = W_x x (``dt_rank``, ``state``, ``state``); dt = softplus(W_dt r + b_dt)
-    [inner]; A = -exp(A_log) [inner, state].  Per channel c and state n, S from zero:
-        S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;   y_c = sum_n S[c, n] C_n + D_c x_c
+    """The selective scan of Mamba.  With h the input: [x | z] = W_in h (``inner`` each); x = silu(conv(x)), a convolution over
+    the last ``conv`` tokens channel by channel, with a bias; [r | B | C] = W_x x (``dt_rank``, ``state``, ``state``); dt = softplus(W_dt r + b_dt)
+    [inner]; A = -exp(A_log) [inner, state].  With S [inner, state] from zero:
+        S <- S * exp(dt[:, None] A) + (dt x) B^T;   y = S C + D * x                 token by token
     then y * silu(z) through W_o.  Step sizes, decays, state and read-out are 32-bit.  ``names``: in, conv, x, dt, A_log, D, o after
     the prefix; the two biases are the convolution's and dt's names plus ``bias_suffix``."""
 
@@ -266,10 +266,10 @@ class SelectiveScanSpec:
 @dataclass(frozen=True)
 class StateSpaceSpec:
     """The state-space recurrence of Mamba-2, one decay per token and head.  With h the input and inner = heads * value_dim:
-    [z: inner | x: inner | B: groups * state | C: groups * state | dt: heads] = W_in h; x, B and C together pass a causal convolution of
-    ``conv`` taps per channel with a bias, and a SiLU; dt = softplus(dt + dt_bias).  Per head (B and C of group h // (heads /
+    [z: inner | x: inner | B: groups * state | C: groups * state | dt: heads] = W_in h; [x | B | C] = silu(conv([x | B | C])), a
+    convolution over the last ``conv`` tokens channel by channel, with a bias; dt = softplus(dt + dt_bias).  Per head (B and C of group h // (heads /
     groups)), S [state, value_dim] from zero:
-        S_t = exp(-exp(A_log_h) dt) S_(t-1) + dt B_t x_t^T;   y_t = S_t^T C_t + D_h x_t
+        S <- S exp(-dt exp(A_log)) + B (dt x)^T;   y = C^T S + D x                  token by token
     then y * silu(z), an RMS norm in ``norm_groups`` equal parts (``norm_eps``) times a weight [inner], through W_o.  Step sizes,
     decays, state and read-out are 32-bit.  ``names``: in, conv, dt_bias, A_log, D, norm, o after the prefix; the convolution's
     bias is its name plus ``bias_suffix``."""
@@ -346,10 +346,10 @@ class MoESpec:
     sigmoid(w h), one number per token, w [1, hidden] this tensor after the shared prefix ("" for none).  The soft-max over the
     chosen logits is the soft-max over all logits divided by the chosen ones' sum.  Experts of the form ``PlainFFSpec`` have no gate
     matrix.
-    ``score`` = "softmax_all": the scores are s = soft-max over all logits; the choice goes by s + correction and the weights are
-    the chosen experts' s divided by their sum (+ 1e-20).  ``group_best`` = 1: a group's score is its largest choice score alone.
+    ``score`` = "softmax_all": the scores are s = soft-max over all logits; the choice goes by s + correction, and what was
+    chosen is weighted by s over the sum of the chosen s (+ 1e-20).  ``group_best`` = 1: a group's score is its largest choice score alone.
     ``weight_scale`` multiplies the weights, whatever the scores.  ``identity``: so many more outputs of the router, behind the
-    experts' (and in the groups and the soft-max with them), are experts without tensors whose output is the input itself."""
+    experts' (and in the groups and the soft-max with them), hand their input back (no matrices)."""
 
     kind: ClassVar[str] = "moe"
     hidden: int

@@ -1,7 +1,7 @@
 // The selective scan of Mamba: a recurrence over the tokens with a state of N numbers per channel, whose step size, input
-// and read-out the tokens choose.  Per channel c and state n, S [inner][N] (a new sequence starts with S = 0):
-//     dt_c  = softplus(zdt_c + bias_c)
-//     S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;    y_c = sum_n S[c, n] C_n + D_c x_c;    out_c = y_c silu(z_c)
+// and read-out the tokens choose.  With S [inner][N] (a new sequence starts with S = 0), token by token, c a channel:
+//     dt[c] = softplus(zdt[c] + bias[c])
+//     S[c] <- S[c] * exp(dt[c] A[c]) + (dt[c] x[c]) B;    y[c] = S[c] . C + D[c] x[c];    out[c] = y[c] silu(z[c])
 // Step sizes, decays, state and read-out are 32-bit.
 //
 // No channel meets another: a channel's states lie in TPC neighbouring lanes, SPT states a lane, whose parts of y meet through

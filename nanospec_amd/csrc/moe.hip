@@ -107,7 +107,7 @@ __global__ __launch_bounds__(256) void moe_logits_few_kernel(const T* __restrict
 // ``score`` = MOE_SIGMOID: scores s = sigmoid(z); the choice goes by s + correction[e] (``correction`` may be null) and the
 // weights are the chosen experts' s, not renormalized.
 // ``score`` = MOE_SOFTMAX: scores s = soft-max over all logits; the choice goes by s + correction[e], the weights are the chosen
-// experts' s divided by their sum (+ 1e-20).
+// s over the sum of the chosen s (+ 1e-20).
 // All weights are then multiplied by ``scale``.  ``groups`` > 1: the experts form that many equal groups of neighbours; a
 // group's score is the sum of its ``group_best`` (1 or 2) largest choice scores (of its one, if it has one), and only the
 // ``keep`` best groups' experts can be chosen: the others never enter the comparison, whatever their scores' sign.

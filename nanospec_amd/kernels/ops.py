@@ -1356,7 +1356,7 @@ SELECTIVE_SCAN_MAX_STATE = 512
 
 class SelectiveRows:
     """The operands of Mamba's selective scan (``selective_scan``, ``selective_chunks``; ``csrc/mamba.hip``): dt = softplus(zdt + dt_bias);
-    S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n; y_c = sum_n S[c, n] C_n + skip_c x_c; out = y silu(z).  ``x`` float32
+    S <- S * exp(dt[:, None] A) + (dt x) B^T; y = S C + skip * x; out = y silu(z).  ``x`` float32
     [tokens, inner]; ``zdt``, ``z`` [tokens, inner] (may be column slices) and ``bc`` (B at the column ``b_off``, C at ``c_off``) in
     the model's dtype, as ``out``; ``A`` float32 [inner, N]; ``state`` float32 [slots, >= inner * N], [inner, N] in a slot."""
 

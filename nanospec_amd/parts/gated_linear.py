@@ -3,9 +3,9 @@ chooses.
 
 h [tokens, hidden] is the mixer's input; H heads, D key channels, E value channels.  Per head:
   q = W_q h * query_scale,  k = W_k h   [D];   v = W_v h   [E];   alpha = sigmoid(W_a2 (W_a1 h) + b)^(1 / tau)   [D]
-  S_t = diag(alpha_t) S_(t-1) + k_t v_t^T;   o_t = S_t^T q_t              S [D, E] starts at zero
+  S <- S * alpha (row by row) + k v^T;   o = q^T S                        token by token, S [D, E] from zero
   y = W_o (o / rms(o) * norm * silu(W_g h))                              rms per head over E, one weight [E] for all heads
-S lives in 32-bit in the request's state slot and is carried from step to step.
+The request's state slot keeps S, in 32-bit.
 
 One product reads h for q, k, v, the gate and W_a1 together (the matrices are stacked at load time), a second one takes the
 thin result through W_a2.  The logarithms of the decays and 32-bit rows of q, k and v (``retention_prep``), the recurrence and the gated

@@ -3,7 +3,7 @@
 h [tokens, hidden] is the mixer's input; c channels (inner), N states a channel, R the rank of the step sizes, K taps.
   [x | z] = W_in h;   x = silu(conv(x) + b)                                short causal convolution per channel
   [r: R | B: N | C: N] = W_x x;   dt = softplus(W_dt r + b_dt)   [c];   A = -exp(A_log)   [c, N]
-  S[c, n] <- exp(dt_c A[c, n]) S[c, n] + dt_c x_c B_n;   y_c = sum_n S[c, n] C_n + D_c x_c       S starts at zero
+  S <- S * exp(dt[:, None] A) + (dt x) B^T;   y = S C + D * x             token by token, S [c, N] from zero
   y = W_o (y * silu(z))
 Three products (h, x, r), the convolution with its carried inputs (``conv_silu_carry``) and one kernel from the step sizes to
 the gated read-out (``selective_scan``; long portions of few states in chunks, ``selective_chunks``); what is not a product is 32-bit.  What a request carries from step to step lives

@@ -1,9 +1,9 @@
 """The state-space recurrence of Mamba-2, one decay per token and head ("state_space").
 
 h [tokens, hidden] is the mixer's input; H heads of E channels (inner = H E), N states, G groups, K taps.
-  [z: inner | x: inner | B: G N | C: G N | dt: H] = W_in h;   [x | B | C] = silu(conv([x | B | C]) + b)
+  [z | x | B | C | dt] = W_in h, of inner, inner, G N, G N and H;   [x | B | C] = silu(conv([x | B | C]) + b)
   dt = softplus(dt + dt_bias)   [H];   log a = -exp(A_log) dt
-  S_t = a_t S_(t-1) + dt_t B_t x_t^T;   y_t = S_t^T C_t + D x_t            per head, B and C of its group; S [N, E] starts at zero
+  S <- a S + B (dt x)^T;   y = C^T S + D x                                 per head, B and C of its group; S [N, E] from zero
   y = W_o (rms(y * silu(z)) * norm)                                       rms in norm_groups equal parts of the inner channels
 One product reads h for everything.  The convolution with its carried inputs (``conv_silu_carry``) leaves 32-bit rows [x | B | C],
 in which the recurrence finds its keys (B), queries (C) and values (x): it is retention's with one decay per token and head

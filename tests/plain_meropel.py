@@ -36,7 +36,7 @@ def pair_rows(tokens: torch.Tensor, buckets: int, mul_prev: int, mul_cur: int) -
 
 def rotate(x: torch.Tensor, positions: torch.Tensor, dims: int, base: float, interleaved: bool) -> torch.Tensor:
     """x [tokens, heads, >= dims]: pair i is channels (i, i + dims / 2), or (2i, 2i + 1) if ``interleaved``; at position p the
-    pair (u, v) becomes (u cos a - v sin a, v cos a + u sin a), a = p base^(-2i / dims)."""
+    pair, read as a complex number, is multiplied by exp(i a), a = p base^(-2i / dims)."""
     out = x.clone()
     for i in range(dims // 2):
         a, b = (2 * i, 2 * i + 1) if interleaved else (i, i + dims // 2)
@@ -82,7 +82,7 @@ def normed_attention(h: torch.Tensor, w: dict, p: str, m: dict, eps: float) -> t
 
 
 def causal_conv(x: torch.Tensor, taps: torch.Tensor, bias: torch.Tensor) -> torch.Tensor:
-    """Per channel sum_j taps[:, j] x[t - (K - 1) + j] + bias, zeros before the start.  x [T, C], taps [C, K]."""
+    """Per channel sum_j taps[:, j] x[t - (K - 1) + j] + bias, what lies in front of the first token counts as nothing.  x [T, C], taps [C, K]."""
     K = taps.shape[1]
     out = bias.expand_as(x).clone()
     for j in range(K):
